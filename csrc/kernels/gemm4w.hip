@@ -16,11 +16,11 @@
 // Per K tile (BK = 64) and wave: 16 NT MFMAs (8 m x NT n tiles x 2 k-steps of 32), 2 (8 + NT)
 // ds_read_b128 fragment reads, 8 + NT LDS-DMA pieces of 1 KiB (the workgroup moves the A | W tile).  LDS
 // holds two K tiles.  Register fragments are double-buffered by k-step: X = k-step 0, Y = k-step 1.  The main
-// loop (G4_TILE_H, hipBLASLt's MT256x256x64 segment shape): seg A = the Y reads of tile R, one
-// per k-step-0 MFMA, lgkmcnt(0), barrier; seg B = the rest of k-step 0 and most of k-step 1, carrying tile
-// R+2's DMA pieces one per ~5 MFMAs at raised wave priority, counted vmcnt, barrier; seg C = the last
-// k-step-1 MFMAs with the X reads of tile R+1.  vmcnt never reaches 0 inside the loop except for the last
-// two tiles.
+// loop (G4_TILE) has three segments per K tile, each load spread evenly over its segment's MFMAs: seg A = all of
+// k-step 0, carrying the Y reads of tile R over its first three quarters (the last quarter covers their latency),
+// lgkmcnt(0), barrier; seg B = the first kSegB MFMAs of k-step 1, carrying tile R+2's DMA pieces, counted vmcnt,
+// barrier; seg C = the rest of k-step 1 with the X reads of tile R+1.  vmcnt never reaches 0 inside the loop except
+// for the last two tiles.
 //   hazards: WAR — tile R+2 overwrites buffer R & 1 only after every wave's reads of tile R completed
 //            (lgkmcnt(0) + barrier closing seg A).  RAW — tile R+1 is read in seg C after every wave's
 //            counted vmcnt wait for it (tile R+2's pieces, the youngest, stay in flight) + the barrier
@@ -191,13 +191,11 @@ LWC_DEVICE float erf_as(float x) {
   return copysignf(1.f - y * __expf(-a * a), x);
 }
 LWC_DEVICE float gelu_erf(float x) { return 0.5f * x * (1.f + erf_as(x * 0.70710678118654752f)); }
-// GELU in the tanh form, x * sigmoid(2 sqrt(2/pi) (x + 0.044715 x^3)) — the form hipBLASLt's bias+GELU
-// epilogue computes (the library arm the planner times against): 2 transcendentals + 4 VALU instead of
-// erf_as's 2 + ~12, within 8.1e-3 of the erf form at the bge-large FFN1 shape, the bf16 output's own rounding
+// GELU in the tanh form, x * sigmoid(2 sqrt(2/pi) (x + 0.044715 x^3)), from tanh(z) = 2 sigmoid(2 z) - 1: 2
+// transcendentals + 4 VALU instead of erf_as's 2 + ~12, within 8.1e-3 of the erf form at the bge-large FFN1 shape, the bf16 output's own rounding
 // being 7.8e-3 (ops/gemm_plan.py linear_bias).  The VAR 64 epilogue uses it; the other schedules keep erf.
 // (A degree-7 polynomial of the erf form, clamped at |x| = 4 — no transcendental, 12 VALU — ran FFN1 + GELU
-// 3.5 % slower at config 2's shape; its packed-fp32 form miscompiled inside this epilogue:
-// profiles/round6_ab.md, scripts/probes/pkfma_probe.cpp.)
+// 3.5 % slower at config 2's shape.)
 LWC_DEVICE float gelu_tanh(float x) {
   const float z = x * (1.5957691216f + 0.0713548163f * x * x);
   return x * __builtin_amdgcn_rcpf(1.f + __expf(-z));
@@ -416,53 +414,45 @@ __global__ void __launch_bounds__(256, 1) gemm4w_kernel(Params p) {
     for (int k = 0; k < G::Reads; ++k) rd1(smem, offA0, offB0, xa, xb, k);
 
     constexpr int M1 = 8 * NT;  // MFMAs of one k-step
-    // VAR 32: the library kernel's segment shape (hipBLASLt's MT256x256x64 DTL loop: the same
-    // 128 MFMA / 32 ds_read_b128 / 16 LDS-DMA per K tile, two barriers).  seg A: the Y reads of tile R back
-    // to back, one per k-step-0 MFMA, then a few more MFMAs, lgkmcnt(0), barrier; seg B: the long middle —
-    // the rest of k-step 0 and most of k-step 1 — carrying the tile R+2 DMA pieces one per ~5 MFMAs at raised
-    // wave priority (s_setprio 3), vmcnt, barrier; seg C: the last k-step-1 MFMAs with the X reads of tile
-    // R+1 one per MFMA.  Waits land after sections with no loads of their own in flight behind them.
-    constexpr int HA = G::Reads + M1 / 6;        // seg A MFMAs (k-step 0)
-    constexpr int HC = G::Reads + M1 / 8;        // seg C MFMAs (k-step 1)
-    constexpr int HB = 2 * M1 - HA - HC;          // seg B MFMAs (k-step 0 rest, then k-step 1)
-#define G4_TILE_H(R, STAGE, NEXT)                                                                   \
+    // Loads per MFMA slot: load k of n goes in front of MFMA ceil((k + 1) len / n) - 1 of a segment of len MFMAs, so no
+    // two loads of a wave are closer than the segment allows.
+    auto slot_has = [](int m, int n, int len) { return m * n / len != (m + 1) * n / len; };
+    auto slot_load = [](int m, int n, int len) { return m * n / len; };
+    constexpr int kReadSpan = M1 * 3 / 4;   // seg A: MFMAs that carry the Y reads
+    constexpr int kSegB = M1 * 5 / 8;       // k-step 1: MFMAs that carry the DMA pieces
+    constexpr int kSegC = M1 - kSegB;       // k-step 1: MFMAs that carry the next tile's X reads
+#define G4_TILE(R, STAGE, NEXT)                                                                     \
   {                                                                                                 \
     uint8_t* cur = smem + ((R) & 1) * G::Buf;                                                       \
     uint8_t* nxt = smem + (((R) + 1) & 1) * G::Buf;                                                 \
-    _Pragma("unroll") for (int m = 0; m < HA; ++m) {                                                \
-      if (m < G::Reads) rd1(cur, offA1, offB1, ya, yb, m);                                          \
-      mfma2<TRL>(acc[m / NT][m % NT], xa[m / NT], xb[m % NT]);                                            \
+    _Pragma("unroll") for (int m = 0; m < M1; ++m) {                                                \
+      if (m < kReadSpan && slot_has(m, G::Reads, kReadSpan)) rd1(cur, offA1, offB1, ya, yb, slot_load(m, G::Reads, kReadSpan)); \
+      mfma2<TRL>(acc[m / NT][m % NT], xa[m / NT], xb[m % NT]);                                      \
       __builtin_amdgcn_sched_barrier(0);                                                            \
     }                                                                                               \
     G4_LGKM0();                                                                                     \
     G4_BAR();                                                                                       \
-    if constexpr ((STAGE) != 0) __builtin_amdgcn_s_setprio(3);                                      \
-    _Pragma("unroll") for (int q = 0; q < HB; ++q) {                                                \
+    _Pragma("unroll") for (int m = 0; m < kSegB; ++m) {                                             \
       if constexpr ((STAGE) == 1) {                                                                 \
-        if (q * G::Pieces / HB != (q + 1) * G::Pieces / HB) piece(cur, (R) + 2, q * G::Pieces / HB); \
+        if (slot_has(m, G::Pieces, kSegB)) piece(cur, (R) + 2, slot_load(m, G::Pieces, kSegB));     \
       } else if constexpr ((STAGE) == 2) {                                                          \
-        if (q * G::Pieces / HB != (q + 1) * G::Pieces / HB) npiece(cur, (R) + 2 - nt, q * G::Pieces / HB); \
+        if (slot_has(m, G::Pieces, kSegB)) npiece(cur, (R) + 2 - nt, slot_load(m, G::Pieces, kSegB)); \
       }                                                                                             \
-      const int m = HA + q;                                                                         \
-      if (m < M1)                                                                                   \
-        mfma2<TRL>(acc[m / NT][m % NT], xa[m / NT], xb[m % NT]);                                          \
-      else                                                                                          \
-        mfma2<TRL>(acc[(m - M1) / NT][(m - M1) % NT], ya[(m - M1) / NT], yb[(m - M1) % NT]);              \
+      mfma2<TRL>(acc[m / NT][m % NT], ya[m / NT], yb[m % NT]);                                      \
       __builtin_amdgcn_sched_barrier(0);                                                            \
     }                                                                                               \
     if constexpr ((STAGE) != 0) {                                                                   \
-      __builtin_amdgcn_s_setprio(0);                                                                \
       G4_VM(G::Pieces);                                                                             \
     } else {                                                                                        \
       G4_VM(0);                                                                                     \
     }                                                                                               \
     G4_BAR();                                                                                       \
-    _Pragma("unroll") for (int c = 0; c < HC; ++c) {                                                \
+    _Pragma("unroll") for (int c = 0; c < kSegC; ++c) {                                             \
       if constexpr (NEXT) {                                                                         \
-        if (c < G::Reads) rd1(nxt, offA0, offB0, xa, xb, c);                                        \
+        if (slot_has(c, G::Reads, kSegC)) rd1(nxt, offA0, offB0, xa, xb, slot_load(c, G::Reads, kSegC)); \
       }                                                                                             \
-      const int m = M1 - HC + c;                                                                    \
-      mfma2<TRL>(acc[m / NT][m % NT], ya[m / NT], yb[m % NT]);                                            \
+      const int m = kSegB + c;                                                                      \
+      mfma2<TRL>(acc[m / NT][m % NT], ya[m / NT], yb[m % NT]);                                      \
       __builtin_amdgcn_sched_barrier(0);                                                            \
     }                                                                                               \
   }
@@ -474,14 +464,14 @@ __global__ void __launch_bounds__(256, 1) gemm4w_kernel(Params p) {
       // other variants' tail: a differently shaped tail made the register allocator rotate the accumulators
       // through v_accvgpr_mov copies that read in-flight inline-asm MFMA results.)
       constexpr int TAIL = PAP ? 2 : 0;
-      for (; r + 2 < nt; ++r) G4_TILE_H(r, 1, true)
+      for (; r + 2 < nt; ++r) G4_TILE(r, 1, true)
       if (nt >= 2) {
-        G4_TILE_H(r, TAIL, true)
+        G4_TILE(r, TAIL, true)
         ++r;
       }
-      G4_TILE_H(r, TAIL, false)
+      G4_TILE(r, TAIL, false)
     }
-#undef G4_TILE_H
+#undef G4_TILE
     // accumulators are read by VALU / stores from here on.  The MFMAs are opaque inline asm, so the compiler
     // takes their results as ready at once: without a barrier it hoisted v_accvgpr_read of the last MFMAs'
     // accumulators above the drain (the row-scaled variant read stale e = 2, 3 values).  The drain, then an
