@@ -71,6 +71,10 @@ PER_FILE_FLAGS = {f: ["-mllvm", "-amdgpu-mfma-vgpr-form=1"] for f in ("attention
                                                                       "wattn.hip", "wattn_decode_wide.hip")}
 
 
+# hipcc -O3 forms packed fp32 instructions by itself from scalar float code; this keeps it from doing so
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+
 def build_kernels(jobs: int = 8, force: bool = False) -> Path:
     """Compile every csrc/kernels/*.hip for gfx950 and link the torch extension."""
     kdir = CSRC / "kernels"
@@ -78,7 +82,7 @@ def build_kernels(jobs: int = 8, force: bool = False) -> Path:
     obj_dir.mkdir(parents=True, exist_ok=True)
     headers = sorted(kdir.glob("*.h"))
     hip_srcs = sorted(kdir.glob("*.hip"))
-    base = ["hipcc", f"--offload-arch={ARCH}", "-O3", "-fPIC", "-std=c++17", "-munsafe-fp-atomics",
+    base = ["hipcc", f"--offload-arch={ARCH}", "-O3", "-fPIC", "-std=c++17", "-munsafe-fp-atomics", *NO_PACKED_FP32,
             "-Wno-unused-result", f"-I{kdir}"]
     tflags, tlibs = _torch_flags()
     jobs_list = []
@@ -101,10 +105,6 @@ def build_kernels(jobs: int = 8, force: bool = False) -> Path:
               *tlibs])
         _check_kernel_stubs(KERNELS_SO)
     return KERNELS_SO
-
-
-# hipcc -O3 forms packed fp32 instructions by itself from scalar float code; this keeps it from doing so
-NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def build_res32(jobs: int = 8, force: bool = False) -> Path:
