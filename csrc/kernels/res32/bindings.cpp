@@ -34,7 +34,7 @@ int r32_delta_rule(float*, int, const void*, int, int, int, const float*, const 
                    const int*, const int*, float*, int, int, int, int, int, int, int, int, hipStream_t);
 int r32_head_norm_gate(const float*, int, const void*, int, const float*, void*, int, int, int, int, float, int, int,
                        hipStream_t);
-int r32_embed_rows(const void*, const int*, float*, int, int, int, float, int, hipStream_t);
+int r32_embed_rows(const void*, const int*, float*, int, int, int, float, void*, int, hipStream_t);
 int r32_head_norm_kv_write(const void*, int, int, int, const int*, const int*, float*, void*, void*, long long, long long,
                            int, int, int, int, int, int, float, float, float, int, int, hipStream_t);
 int r32_gate_mul(void*, int, const void*, int, int, int, int, int, hipStream_t);
@@ -46,22 +46,27 @@ int r32_rmsnorm_rows(const float*, const long long*, const float*, void*, int, i
 int r32_gelu_mul_rows(const void*, int, const void*, int, int, const int*, int, void*, int, int, int, hipStream_t);
 int r32_stack_mix(const float*, long long, const float*, int, float*, long long, hipStream_t);
 int r32_router_max_outputs();
-int r32_router(const float*, const float*, const float*, int, int, int, int, int, int*, float*, int*, int*, int*, int*, int*,
-               int*, hipStream_t);
+int r32_router(const float*, int, const float*, const float*, int, int, float, float, int, int, int, int, int, int, int*, float*,
+               int*, int*, int*, int*, int*, int*, hipStream_t);
 int r32_expert_rows(const void*, int, const int*, const int*, const int*, int, const void*, const void*, float*, int, int,
-                    int, int, hipStream_t);
-int r32_moe_combine(const void*, int, const int*, const float*, const void*, int, int, int, float*, int, const void*, int, int,
-                    hipStream_t);
+                    int, int, float, float, int, hipStream_t);
+int r32_moe_combine(const void*, int, const int*, const float*, const void*, int, int, int, float*, int, const void*, int,
+                    const float*, int, int, hipStream_t);
+int r32_post_norm(float*, const void*, int, float, const float*, void*, int, int, float, int, hipStream_t);
+int r32_post_norm_experts_ok(int);
+int r32_post_norm_experts(float*, const void*, const int*, const float*, int, const void*, int, const float*, int, float,
+                          const float*, void*, int, int, float, int, hipStream_t);
+int r32_head_gate_rows(const void*, long long, long long, const void*, int, void*, int, int, int, int, int, hipStream_t);
 int r32_latent_kv_write(const void*, int, int, int, int, const float*, const float*, const float*, float, const int*,
                         const int*, void*, int, void*, void*, long long, long long, int, int, int, float, int, int,
                         hipStream_t);
 int r32_latent_q_rows(const void*, int, int, int, const float*, int, const float*, float, float, const int*, float*, int, int,
                       int, int, hipStream_t);
 int r32_retention_max_dim();
-int r32_retention_prep(const void*, int, int, const float*, float, const int*, float*, int, int, int, int, float, int,
+int r32_retention_prep(const void*, int, int, const float*, float, const int*, float*, int, int, int, int, float, int, int,
                        hipStream_t);
 int r32_retention(const float*, const void*, int, const float*, float*, long long, const int*, const int*, const int*, float*,
-                  int, int, int, int, int, int, hipStream_t);
+                  int, int, int, int, int, int, int, hipStream_t);
 int r32_glu(const void*, int, void*, int, int, int, int, float, float, int, hipStream_t);
 int r32_gelu(const void*, int, void*, int, int, int, int, hipStream_t);
 int r32_rot_kv_write(const void*, int, const float*, const float*, const float*, float, int, const float*, const int*,
@@ -462,14 +467,21 @@ void head_norm_gate(Tensor o, c10::optional<Tensor> gate, c10::optional<Tensor> 
                           stream()), "head_norm_gate");
 }
 
-void embed_rows(Tensor table, Tensor tokens, Tensor out, double scale) {
+// cast (bf16 [T, d], or absent) also receives the rows
+void embed_rows(Tensor table, Tensor tokens, Tensor out, double scale, c10::optional<Tensor> cast) {
   const int f = act_f32(table, "embed_rows table");
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous(), "embed_rows: table [V, d]");
   want(tokens, torch::kInt32, "embed_rows tokens");
   want(out, torch::kFloat32, "embed_rows out");
   const int T = (int)tokens.numel(), d = (int)table.size(1);
   TORCH_CHECK(out.numel() == (int64_t)T * d, "embed_rows: out [T, d]");
-  done(r32_embed_rows(table.data_ptr(), tokens.data_ptr<int>(), out.data_ptr<float>(), T, d, (int)table.size(0), (float)scale, f,
+  void* cp = nullptr;
+  if (cast.has_value()) {
+    want(*cast, torch::kBFloat16, "embed_rows cast");
+    TORCH_CHECK(cast->numel() == out.numel(), "embed_rows: cast [T, d]");
+    cp = cast->data_ptr();
+  }
+  done(r32_embed_rows(table.data_ptr(), tokens.data_ptr<int>(), out.data_ptr<float>(), T, d, (int)table.size(0), (float)scale, cp, f,
                       stream()), "embed_rows");
 }
 
@@ -585,17 +597,21 @@ void stack_mix(Tensor X, Tensor coef, int64_t n, Tensor out) {
 
 int64_t router_max_outputs() { return r32_router_max_outputs(); }
 
-// z fp32 [T, NE] router logits, corr fp32 [NE]; the first E outputs are real experts.  Returns
+// z fp32 [T, NE] router logits (a column slice is fine), corr fp32 [NE]; the first E outputs are real experts.  Returns
 // (ids [T,k] i32, w [T,k] f32, row_off [E+1] i32, src [T*k] i32, row_expert [T*k] i32, inv [T*k] i32).
-// bias fp32 [NE] is added to the logits; renorm: the chosen weights are divided by their sum (= softmax over the chosen).
+// bias fp32 [NE] is added to the logits; sigmoid: scores = sigmoid(z), else the softmax; renorm: the chosen weights are
+// divided by their sum + floor, then times scale; groups > 1: only outputs of the `keep` best groups may be chosen.
 std::vector<Tensor> router(Tensor z, c10::optional<Tensor> corr, int64_t E, int64_t k, c10::optional<Tensor> bias,
-                           bool renorm) {
-  want(z, torch::kFloat32, "router z");
+                           bool renorm, bool sigmoid, double floor, double scale, int64_t groups, int64_t keep) {
+  want_dev(z, torch::kFloat32, "router z");
+  const int ldz = row_stride(z, "router z");
   if (corr.has_value()) want(*corr, torch::kFloat32, "router correction");
   if (bias.has_value()) want(*bias, torch::kFloat32, "router bias");
   TORCH_CHECK(z.dim() == 2 && (!corr.has_value() || corr->numel() == z.size(1)) &&
                   (!bias.has_value() || bias->numel() == z.size(1)) && E >= 0 && E <= z.size(1) && k >= 1 && k <= z.size(1) &&
                   z.size(1) <= r32_router_max_outputs(), "router: shapes disagree");
+  TORCH_CHECK(groups <= 1 || (z.size(1) % groups == 0 && keep >= 1 && keep <= groups && k <= keep * (z.size(1) / groups)),
+              "router: groups");
   const int T = (int)z.size(0), NE = (int)z.size(1);
   auto oi = z.options().dtype(torch::kInt32);
   Tensor ids = torch::empty({T, k}, oi), w = torch::empty({T, k}, z.options()), rank = torch::empty({T, k}, oi);
@@ -603,8 +619,9 @@ std::vector<Tensor> router(Tensor z, c10::optional<Tensor> corr, int64_t E, int6
   Tensor zeroed = torch::zeros({Ec + 2 * (int64_t)T * k}, oi);  // counts | src | row_expert: one fill
   Tensor counts = zeroed.narrow(0, 0, Ec), src = zeroed.narrow(0, Ec, T * k), row_expert = zeroed.narrow(0, Ec + T * k, T * k);
   Tensor row_off = torch::empty({E + 1}, oi), inv = torch::empty({T * k}, oi);
-  done(r32_router(z.data_ptr<float>(), corr.has_value() ? corr->data_ptr<float>() : nullptr,
-                  bias.has_value() ? bias->data_ptr<float>() : nullptr, renorm ? 1 : 0, T, NE, (int)E, (int)k, ids.data_ptr<int>(), w.data_ptr<float>(),
+  done(r32_router(z.data_ptr<float>(), ldz, corr.has_value() ? corr->data_ptr<float>() : nullptr,
+                  bias.has_value() ? bias->data_ptr<float>() : nullptr, sigmoid ? 1 : 0, renorm ? 1 : 0, (float)floor, (float)scale,
+                  (int)groups, (int)keep, T, NE, (int)E, (int)k, ids.data_ptr<int>(), w.data_ptr<float>(),
                   counts.data_ptr<int>(), rank.data_ptr<int>(), row_off.data_ptr<int>(), src.data_ptr<int>(),
                   row_expert.data_ptr<int>(), inv.data_ptr<int>(), stream()), "router");
   if (T == 0) row_off.zero_();
@@ -612,8 +629,9 @@ std::vector<Tensor> router(Tensor z, c10::optional<Tensor> corr, int64_t E, int6
 }
 
 // h [T, d]; w_gu [E, 2 ff, d] (gate rows, then up rows), w_down [E, d, ff]; returns Y fp32 [len(src), d] (rows beyond
-// row_off[E] are not written)
-Tensor expert_rows(Tensor h, Tensor src, Tensor row_expert, Tensor row_off, Tensor w_gu, Tensor w_down) {
+// row_off[E] are not written).  clamped: the clamped gate unit with alpha and limit, else silu(g) u
+Tensor expert_rows(Tensor h, Tensor src, Tensor row_expert, Tensor row_off, Tensor w_gu, Tensor w_down, bool clamped, double alpha,
+                   double limit) {
   const int f = act_f32(h, "expert_rows h");
   const int ldh = row_stride(h, "expert_rows h");
   want(src, torch::kInt32, "expert_rows src");
@@ -627,13 +645,23 @@ Tensor expert_rows(Tensor h, Tensor src, Tensor row_expert, Tensor row_off, Tens
   Tensor Y = torch::empty({src.numel(), d}, h.options().dtype(torch::kFloat32));
   done(r32_expert_rows(h.data_ptr(), ldh, src.data_ptr<int>(), row_expert.data_ptr<int>(), row_off.data_ptr<int>(),
                        (int)w_gu.size(0), w_gu.data_ptr(), w_down.data_ptr(), Y.data_ptr<float>(), (int)src.numel(), d,
-                       (int)w_down.size(2), f, stream()), "expert_rows");
+                       (int)w_down.size(2), clamped ? 1 : 0, (float)alpha, (float)limit, f, stream()), "expert_rows");
   return Y;
 }
 
 // out fp32 [T, d] = sum_j w[t][j] * (inv[t k + j] >= 0 ? Y[inv] : h[t])
-// add: rows [T, d] of h's dtype added to every token's sum (a shared expert's result), or absent
-Tensor moe_combine(Tensor Y, Tensor inv, Tensor w, Tensor h, c10::optional<Tensor> add) {
+// fp32 logits, one per token, that gate an added row (element t at t * stride); null when absent
+const float* row_gate(const c10::optional<Tensor>& g, int T, int& ld, const char* what) {
+  ld = 0;
+  if (!g.has_value()) return nullptr;
+  TORCH_CHECK(g->is_cuda() && g->scalar_type() == torch::kFloat32 && g->dim() == 1 && g->size(0) == T, what, ": gate fp32 [T]");
+  ld = (int)g->stride(0);
+  return g->data_ptr<float>();
+}
+
+// add: rows [T, d] of h's dtype added to every token's sum (a shared expert's result), or absent; gate: fp32 [T] logits
+// whose sigmoid multiplies them, or absent
+Tensor moe_combine(Tensor Y, Tensor inv, Tensor w, Tensor h, c10::optional<Tensor> add, c10::optional<Tensor> gate) {
   const int f = act_f32(h, "moe_combine h"), fy = act_f32(Y, "moe_combine Y");
   const int ldh = row_stride(h, "moe_combine h");
   want(inv, torch::kInt32, "moe_combine inv");
@@ -650,18 +678,83 @@ Tensor moe_combine(Tensor Y, Tensor inv, Tensor w, Tensor h, c10::optional<Tenso
     lda = row_stride(*add, "moe_combine add");
     ap = add->data_ptr();
   }
+  int ldg = 0;
+  const float* gp = row_gate(gate, T, ldg, "moe_combine");
   done(r32_moe_combine(Y.data_ptr(), fy, inv.data_ptr<int>(), w.data_ptr<float>(), h.data_ptr(), ldh, T, (int)w.size(1),
-                       out.data_ptr<float>(), d, ap, lda, f, stream()), "moe_combine");
+                       out.data_ptr<float>(), d, ap, lda, gp, ldg, f, stream()), "moe_combine");
   return out;
 }
 
+// x fp32 [T, d] <- rms_norm(alpha x + y) * w in place; cast (bf16 [T, d], or absent) also receives the new x
+void* cast_rows(const c10::optional<Tensor>& cast, const Tensor& x, const char* what) {
+  if (!cast.has_value()) return nullptr;
+  want(*cast, torch::kBFloat16, what);
+  TORCH_CHECK(cast->numel() == x.numel(), what, ": [T, d]");
+  return cast->data_ptr();
+}
+
+void post_norm(Tensor x, Tensor y, double alpha, Tensor w, double eps, c10::optional<Tensor> cast) {
+  want(x, torch::kFloat32, "post_norm x");
+  want(w, torch::kFloat32, "post_norm w");
+  const int f = act_f32(y, "post_norm y"), ldy = row_stride(y, "post_norm y");
+  TORCH_CHECK(x.dim() == 2 && y.size(0) == x.size(0) && y.size(1) == x.size(1) && w.numel() == x.size(1), "post_norm: shapes disagree");
+  done(r32_post_norm(x.data_ptr<float>(), y.data_ptr(), ldy, (float)alpha, w.data_ptr<float>(), cast_rows(cast, x, "post_norm cast"),
+                     (int)x.size(0), (int)x.size(1), (float)eps, f, stream()), "post_norm");
+}
+
+bool post_norm_experts_ok(int64_t d) { return r32_post_norm_experts_ok((int)d) != 0; }
+
+// y = sum_j w[t][j] Y[inv[t k + j]] + sigmoid(gate[t]) shared[t], then as post_norm; Y fp32 or bf16 [rows, d]
+void post_norm_experts(Tensor x, Tensor Y, Tensor inv, Tensor wts, c10::optional<Tensor> shared, c10::optional<Tensor> gate,
+                       double alpha, Tensor w, double eps, c10::optional<Tensor> cast) {
+  want(x, torch::kFloat32, "post_norm_experts x");
+  want(w, torch::kFloat32, "post_norm_experts w");
+  want(inv, torch::kInt32, "post_norm_experts inv");
+  want(wts, torch::kFloat32, "post_norm_experts weights");
+  const int fy = act_f32(Y, "post_norm_experts Y");
+  const int T = (int)x.size(0), d = (int)x.size(1);
+  TORCH_CHECK(x.dim() == 2 && Y.is_contiguous() && Y.dim() == 2 && Y.size(1) == d && wts.dim() == 2 && wts.size(0) == T &&
+                  inv.numel() == wts.numel() && Y.size(0) >= inv.numel() && w.numel() == d, "post_norm_experts: shapes disagree");
+  const void* sp = nullptr;
+  int lds = 0, fs = fy, ldg = 0;
+  if (shared.has_value()) {
+    fs = act_f32(*shared, "post_norm_experts shared");
+    lds = row_stride(*shared, "post_norm_experts shared");
+    TORCH_CHECK(shared->size(0) == T && shared->size(1) == d, "post_norm_experts: shared [T, d]");
+    sp = shared->data_ptr();
+  }
+  const float* gp = row_gate(gate, T, ldg, "post_norm_experts");
+  done(r32_post_norm_experts(x.data_ptr<float>(), Y.data_ptr(), inv.data_ptr<int>(), wts.data_ptr<float>(), (int)wts.size(1), sp,
+                             lds, gp, ldg, (float)alpha, w.data_ptr<float>(), cast_rows(cast, x, "post_norm_experts cast"), T, d,
+                             (float)eps, fy | (fs << 1), stream()), "post_norm_experts");
+}
+
+// o [T, H, Dv] (unit last stride, any others), gate [T, H] logits (a column slice is fine), out [T, H Dv]
+void head_gate_rows(Tensor o, Tensor gate, Tensor out) {
+  const int f = act_f32(o, "head_gate_rows o");
+  const int ldg = row_stride(gate, "head_gate_rows gate"), ldo = row_stride(out, "head_gate_rows out");
+  TORCH_CHECK(o.is_cuda() && o.dim() == 3 && (o.stride(2) == 1 || o.size(2) == 1) && gate.scalar_type() == o.scalar_type() &&
+                  out.scalar_type() == o.scalar_type() && gate.is_cuda() && out.is_cuda(), "head_gate_rows: dtypes");
+  const int T = (int)o.size(0), H = (int)o.size(1), Dv = (int)o.size(2);
+  TORCH_CHECK(gate.size(0) == T && gate.size(1) == H && out.size(0) == T && out.size(1) == (int64_t)H * Dv, "head_gate_rows: shapes");
+  done(r32_head_gate_rows(o.data_ptr(), (long long)o.stride(0), (long long)o.stride(1), gate.data_ptr(), ldg, out.data_ptr(), ldo, T,
+                          H, Dv, f, stream()), "head_gate_rows");
+}
+
 // Low-rank attention, cache side: proj rows [dq (Cq) | c (C) | rotated key part (R) | ...]; cq [T, Cq] receives the
-// normalised query latent; the normalised c and the rotated part go to the K row (zeros up to nk), c again to the V row.
-void latent_kv_write(Tensor proj, int64_t Cq, int64_t C, int64_t R, Tensor wq, Tensor wc, Tensor freq, double mult,
-                     Tensor positions, Tensor slots, Tensor cq, Tensor k_cache, Tensor v_cache, double eps) {
+// normalised query latent (Cq = 0: none, wq and cq absent); the normalised c and the rotated part go to the K row (zeros
+// up to nk), c again to the V row.
+void latent_kv_write(Tensor proj, int64_t Cq, int64_t C, int64_t R, c10::optional<Tensor> wq, Tensor wc, Tensor freq, double mult,
+                     Tensor positions, Tensor slots, c10::optional<Tensor> cq, Tensor k_cache, Tensor v_cache, double eps) {
   const int f = act_f32(proj, "latent_kv_write proj");
-  const int ldp = row_stride(proj, "latent_kv_write proj"), ldq = row_stride(cq, "latent_kv_write cq");
-  want(wq, torch::kFloat32, "latent_kv_write wq");
+  const int ldp = row_stride(proj, "latent_kv_write proj");
+  TORCH_CHECK(Cq >= 0 && (Cq == 0 || (wq.has_value() && cq.has_value())), "latent_kv_write: query latent");
+  const int ldq = Cq ? row_stride(*cq, "latent_kv_write cq") : 0;
+  if (Cq) {
+    want(*wq, torch::kFloat32, "latent_kv_write wq");
+    TORCH_CHECK(cq->is_cuda() && cq->scalar_type() == proj.scalar_type() && cq->size(0) == proj.size(0) && cq->size(1) == Cq &&
+                    wq->numel() == Cq, "latent_kv_write: cq");
+  }
   want(wc, torch::kFloat32, "latent_kv_write wc");
   want(freq, torch::kFloat32, "latent_kv_write freq");
   want(positions, torch::kInt32, "latent_kv_write positions");
@@ -669,15 +762,13 @@ void latent_kv_write(Tensor proj, int64_t Cq, int64_t C, int64_t R, Tensor wq, T
   int NB, BS, nk, nv;
   cache_layout(k_cache, v_cache, NB, BS, nk, nv, "latent_kv_write");
   const int T = (int)proj.size(0);
-  TORCH_CHECK(k_cache.scalar_type() == proj.scalar_type() && v_cache.scalar_type() == proj.scalar_type() &&
-                  cq.scalar_type() == proj.scalar_type() && cq.is_cuda() && k_cache.is_cuda() && v_cache.is_cuda(),
-              "latent_kv_write: one activation dtype");
-  TORCH_CHECK(Cq >= 1 && C >= 1 && R >= 0 && R % 2 == 0 && proj.size(1) >= Cq + C + R && cq.size(0) == T && cq.size(1) == Cq &&
-                  wq.numel() == Cq && wc.numel() == C && freq.numel() == R / 2 && positions.numel() == T && slots.numel() == T &&
+  TORCH_CHECK(k_cache.scalar_type() == proj.scalar_type() && v_cache.scalar_type() == proj.scalar_type() && k_cache.is_cuda() &&
+                  v_cache.is_cuda(), "latent_kv_write: one activation dtype");
+  TORCH_CHECK(C >= 1 && R >= 0 && R % 2 == 0 && proj.size(1) >= Cq + C + R && wc.numel() == C && freq.numel() == R / 2 && positions.numel() == T && slots.numel() == T &&
                   nk >= C + R && nv >= C, "latent_kv_write: shapes disagree");
-  done(r32_latent_kv_write(proj.data_ptr(), ldp, (int)Cq, (int)C, (int)R, wq.data_ptr<float>(), wc.data_ptr<float>(),
-                           freq.data_ptr<float>(), (float)mult, positions.data_ptr<int>(), slots.data_ptr<int>(), cq.data_ptr(),
-                           ldq, k_cache.data_ptr(), v_cache.data_ptr(), (long long)k_cache.stride(0),
+  done(r32_latent_kv_write(proj.data_ptr(), ldp, (int)Cq, (int)C, (int)R, Cq ? wq->data_ptr<float>() : nullptr,
+                           wc.data_ptr<float>(), freq.data_ptr<float>(), (float)mult, positions.data_ptr<int>(),
+                           slots.data_ptr<int>(), Cq ? cq->data_ptr() : nullptr, ldq, k_cache.data_ptr(), v_cache.data_ptr(), (long long)k_cache.stride(0),
                            (long long)v_cache.stride(0), BS, nk, nv, (float)eps, T, f, stream()), "latent_kv_write");
 }
 
@@ -738,9 +829,9 @@ void latent_expand_write(Tensor kv, Tensor lat, int64_t rot_off, int64_t R, Tens
 int64_t retention_max_dim() { return r32_retention_max_dim(); }
 
 // proj rows with q at column 0 and k at k_off (H heads of D each); v rows [T, H Dv] (a column slice is fine); state fp32
-// [slots, H, D, Dv]; out fp32 [T, H Dv]
+// [slots, H, D, Dv]; out fp32 [T, H Dv]; k_scale multiplies k; act: q, k and v go through silu first
 void retention(Tensor proj, int64_t k_off, Tensor v, Tensor freq, double mult, int64_t rd, Tensor decay, Tensor state, Tensor cu,
-               Tensor item_slot, Tensor positions, Tensor out, int64_t H) {
+               Tensor item_slot, Tensor positions, Tensor out, int64_t H, double k_scale, bool act) {
   const int f = act_f32(proj, "retention proj");
   const int ldp = row_stride(proj, "retention proj"), ldv = row_stride(v, "retention v"), ldo = row_stride(out, "retention out");
   want(freq, torch::kFloat32, "retention freq");
@@ -760,11 +851,11 @@ void retention(Tensor proj, int64_t k_off, Tensor v, Tensor freq, double mult, i
               "retention: shapes disagree");
   Tensor qk = torch::empty({T, 2 * H * D}, out.options());
   done(r32_retention_prep(proj.data_ptr(), ldp, (int)k_off, freq.data_ptr<float>(), (float)mult, positions.data_ptr<int>(),
-                          qk.data_ptr<float>(), T, (int)H, D, (int)rd, 1.0f / std::sqrt((float)D), f, stream()),
+                          qk.data_ptr<float>(), T, (int)H, D, (int)rd, (float)k_scale, act ? 1 : 0, f, stream()),
        "retention_prep");
   done(r32_retention(qk.data_ptr<float>(), v.data_ptr(), ldv, decay.data_ptr<float>(), state.data_ptr<float>(),
                      (long long)state.stride(0), cu.data_ptr<int>(), item_slot.data_ptr<int>(), positions.data_ptr<int>(),
-                     out.data_ptr<float>(), ldo, (int)item_slot.numel(), (int)H, D, Dv, f, stream()), "retention");
+                     out.data_ptr<float>(), ldo, (int)item_slot.numel(), (int)H, D, Dv, act ? 1 : 0, f, stream()), "retention");
 }
 
 // in rows [gate (n) | up (n)], out rows of n; mode 0 silu(g) u, 1 the clamped unit g' sigmoid(alpha g') (u' + 1)
@@ -935,6 +1026,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("router_max_outputs", &router_max_outputs);
   m.def("expert_rows", &expert_rows);
   m.def("moe_combine", &moe_combine);
+  m.def("post_norm", &post_norm);
+  m.def("post_norm_experts", &post_norm_experts);
+  m.def("post_norm_experts_ok", &post_norm_experts_ok);
+  m.def("head_gate_rows", &head_gate_rows);
   m.def("latent_kv_write", &latent_kv_write);
   m.def("latent_q_rows", &latent_q_rows);
   m.def("latent_expand_write", &latent_expand_write);

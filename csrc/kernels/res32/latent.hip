@@ -7,9 +7,13 @@
 // one row (key size C + R, value size C), which the window_attn kernels run with G = 1.
 //
 //   latent_kv_write   from fused projection rows [ dq (Cq) | dkv (C + R) | ... ]: cq = dq / rms(dq) * wq -> rows of the
-//                     activation type; c = dkv[:C] / rms * wc and the rotated rest -> the paged cache
+//                     activation type (Cq = 0: queries without a latent, nothing to do); c = dkv[:C] / rms * wc and the
+//                     rotated rest -> the paged cache
 //   latent_q_rows     the fp32 query rows [ qn * scale (C) | rot(q_rot) * scale (R) | 0 ] per head from the absorbed
 //                     unrotated part qn ([H, T, C] fp32) and the up-projected query rows (rotated part of every head)
+//
+//   head_gate_rows    out[t, h, :] = o[t, h, :] * sigmoid(gate[t, h]): one gate per head on the attention's result, from
+//                     whatever strides the up-projection left it in ([H, T, Dv] of a batched product, padded heads)
 //
 // Rotation ("interleaved"): entries (2i, 2i + 1) at position p turn by the angle a = p * f_i (fp32 product of the
 // position and the fp32 frequency), (u, v) -> m (u cos a - v sin a, v cos a + u sin a); f and m come from the host
@@ -38,7 +42,7 @@ latent_kv_write_kernel(const AT* __restrict__ proj, int ldp, int Cq, int C, int 
     const float x = Elem<AT>::ld(pr + Cq + i);
     sc += x * x;
   }
-  const float rq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)Cq + eps);
+  const float rq = Cq > 0 ? 1.0f / sqrtf(block_sum(sq, scratch) / (float)Cq + eps) : 0.f;
   const float rc = 1.0f / sqrtf(block_sum(sc, scratch) / (float)C + eps);
   for (int i = threadIdx.x; i < Cq; i += blockDim.x)
     Elem<AT>::st(cq + (size_t)t * ldq + i, Elem<AT>::ld(pr + i) * rq * wq[i]);
@@ -125,10 +129,56 @@ latent_expand_write_kernel(const AT* __restrict__ kv, int ldk, const AT* __restr
   }
 }
 
+template <typename AT>
+__global__ void __launch_bounds__(256) head_gate_rows_kernel(const AT* __restrict__ o, long long row_stride, long long head_stride,
+                                                              const AT* __restrict__ gate, int ldg, AT* __restrict__ out, int ldo,
+                                                              int H, int Dv) {
+  const int t = blockIdx.x;
+  for (int e = threadIdx.x; e < H * Dv; e += blockDim.x) {
+    const int h = e / Dv, i = e - h * Dv;
+    const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + h));
+    Elem<AT>::st(out + (size_t)t * ldo + e, Elem<AT>::ld(o + t * row_stride + h * head_stride + i) * g);
+  }
+}
+
+// four entries per thread: Dv, every stride and every base a multiple of four entries
+template <typename AT>
+__global__ void __launch_bounds__(256) head_gate_rows_vec_kernel(const AT* __restrict__ o, long long row_stride,
+                                                                  long long head_stride, const AT* __restrict__ gate, int ldg,
+                                                                  AT* __restrict__ out, int ldo, int H, int dv4) {
+  const int t = blockIdx.x;
+  for (int e = threadIdx.x; e < H * dv4; e += blockDim.x) {
+    const int h = e / dv4, i = 4 * (e - h * dv4);
+    const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + h));
+    Vec4<AT>::st(out + (size_t)t * ldo + 4 * e, Vec4<AT>::ld(o + t * row_stride + h * head_stride + i) * g);
+  }
+}
+
 }  // namespace
 }  // namespace lwc
 
 using namespace lwc;
+
+extern "C" int r32_head_gate_rows(const void* o, long long row_stride, long long head_stride, const void* gate, int ldg, void* out,
+                                  int ldo, int T, int H, int Dv, int f32, hipStream_t s) {
+  if (T <= 0) return 0;
+  const int ab = f32 ? 16 : 8;
+  const bool vec = Dv % 4 == 0 && row_stride % 4 == 0 && head_stride % 4 == 0 && ldo % 4 == 0 && aligned_to(o, ab) && aligned_to(out, ab);
+#define LWC_HGR(AT)                                                                                                        \
+  if (vec)                                                                                                                 \
+    head_gate_rows_vec_kernel<AT><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, \
+                                                    ldo, H, Dv / 4);                                                       \
+  else                                                                                                                     \
+    head_gate_rows_kernel<AT><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, ldo, H, Dv)
+  if (f32) {
+    LWC_HGR(float);
+  } else {
+    LWC_HGR(bf16_t);
+  }
+#undef LWC_HGR
+  LWC_CHECK_LAUNCH();
+  return 0;
+}
 
 extern "C" int r32_latent_expand_write(const void* kv, int ldk, const void* lat, int ldl, int rot_off, const long long* slots,
                                        void* k_cache, void* v_cache, long long kb_stride, long long vb_stride, int block_size,
@@ -152,7 +202,7 @@ extern "C" int r32_latent_kv_write(const void* proj, int ldp, int Cq, int C, int
                                    void* k_cache, void* v_cache, long long kb_stride, long long vb_stride, int block_size,
                                    int nk, int nv, float eps, int T, int f32, hipStream_t s) {
   if (T <= 0) return 0;
-  if (R % 2 != 0 || nk < C + R || nv < C || Cq < 1 || C < 1) return -1;
+  if (R % 2 != 0 || nk < C + R || nv < C || Cq < 0 || C < 1) return -1;
   if (f32)
     latent_kv_write_kernel<float><<<T, 256, 0, s>>>((const float*)proj, ldp, Cq, C, R, wq, wc, freq, mult, positions, slots,
                                                     (float*)cq, ldq, (float*)k_cache, (float*)v_cache, kb_stride, vb_stride,

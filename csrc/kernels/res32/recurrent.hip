@@ -12,7 +12,7 @@
 //                       S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //                     q, k made unit vectors per head (1e-6 inside the root), q times D^-1/2;
 //                     beta = sigmoid(b), g = exp(-exp(A_log) softplus(a + dt_bias)); state fp32 [slot][H][D][Dv]
-//   head_norm_gate    o / rms(o) over each head's Dv * w * silu(gate) (or sigmoid(gate), or no gate)
+//   head_norm_gate    o / rms(o) over each head's Dv * w * silu(gate) (or sigmoid(gate), or no gate); H = 1: over the row
 #include "elem.h"
 
 namespace lwc {
@@ -362,6 +362,40 @@ __global__ void head_norm_gate_vec_kernel(const float* __restrict__ o, int ldi, 
   }
 }
 
+// One head as wide as the row (a norm over all heads together): the workgroup shares the row, which stays in registers
+// between the sum and the write.  Dv <= 1024 NCH, a multiple of four, aligned bases.
+template <typename AT, int GATE, int NCH>
+__global__ void __launch_bounds__(256) row_norm_gate_kernel(const float* __restrict__ o, int ldi, const AT* __restrict__ gate,
+                                                             int ldg, const float* __restrict__ w, AT* __restrict__ out, int ldo,
+                                                             int Dv, float eps) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  const float* orow = o + (size_t)t * ldi;
+  float4v v[NCH];
+  float s = 0.f;
+#pragma unroll
+  for (int u = 0; u < NCH; ++u) {
+    const int i = (threadIdx.x + 256 * u) * 4;
+    v[u] = i < Dv ? Vec4<float>::ld(orow + i) : float4v{0.f, 0.f, 0.f, 0.f};
+    s += v[u][0] * v[u][0] + v[u][1] * v[u][1] + v[u][2] * v[u][2] + v[u][3] * v[u][3];
+  }
+  const float rstd = 1.0f / sqrtf(block_sum(s, scratch) / (float)Dv + eps);
+#pragma unroll
+  for (int u = 0; u < NCH; ++u) {
+    const int i = (threadIdx.x + 256 * u) * 4;
+    if (i < Dv) {
+      float4v y = v[u] * rstd;
+      if (w) y *= Vec4<float>::ld(w + i);
+      if (GATE) {
+        const float4v z = Vec4<AT>::ld(gate + (size_t)t * ldg + i);
+        y *= GATE == 1 ? float4v{silu_f(z[0]), silu_f(z[1]), silu_f(z[2]), silu_f(z[3])}
+                       : float4v{sigmoid_f(z[0]), sigmoid_f(z[1]), sigmoid_f(z[2]), sigmoid_f(z[3])};
+      }
+      Vec4<AT>::st(out + (size_t)t * ldo + i, y);
+    }
+  }
+}
+
 // Dv / 4 a power of two <= 64: LPH = Dv / 4 lanes per head, 64 / LPH heads per wave at once, every lane busy
 template <typename AT, int GATE>
 __global__ void head_norm_gate_sub_kernel(const float* __restrict__ o, int ldi, const AT* __restrict__ gate, int ldg,
@@ -523,8 +557,18 @@ extern "C" int r32_head_norm_gate(const float* o, int ldi, const void* gate, int
                    aligned_to(gate, ab) && aligned_to(out, ab);
   const int lph = Dv / 4;
   const bool sub = vec && lph >= 1 && lph <= 64 && (lph & (lph - 1)) == 0;
+  const bool row = vec && H == 1 && Dv > 256 && Dv <= 8192;
+#define LWC_RNG(AT, GM, N) row_norm_gate_kernel<AT, GM, N><<<T, 256, 0, s>>>(o, ldi, (const AT*)gate, ldg, w, (AT*)out, ldo, Dv, eps)
 #define LWC_HNG(AT, GM)                                                                                                  \
-  if (sub)                                                                                                               \
+  if (row && Dv <= 1024)                                                                                                 \
+    LWC_RNG(AT, GM, 1);                                                                                                  \
+  else if (row && Dv <= 2048)                                                                                            \
+    LWC_RNG(AT, GM, 2);                                                                                                  \
+  else if (row && Dv <= 4096)                                                                                            \
+    LWC_RNG(AT, GM, 4);                                                                                                  \
+  else if (row)                                                                                                          \
+    LWC_RNG(AT, GM, 8);                                                                                                  \
+  else if (sub)                                                                                                          \
     head_norm_gate_sub_kernel<AT, GM><<<T, threads, 0, s>>>(o, ldi, (const AT*)gate, ldg, w, (AT*)out, ldo, H, Dv, eps,  \
                                                             lph);                                                        \
   else if (vec)                                                                                                          \
@@ -549,6 +593,7 @@ extern "C" int r32_head_norm_gate(const float* o, int ldi, const void* gate, int
     }
   }
 #undef LWC_HNG
+#undef LWC_RNG
   LWC_CHECK_LAUNCH();
   return 0;
 }

@@ -3,8 +3,9 @@
 //   S_t = a_h S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t          S fp32 [D, Dv] per head and sequence
 // q and k are rotated by position on their first `rd` entries ("rotate half": entry i pairs with i + rd / 2, angle
 // p * f_i as an fp32 product), k is then multiplied by D^-1/2.  Everything that enters the recurrence is fp32.
+// Lightning form: q, k and v go through silu first, no rotation (rd = 0), no scale.
 //
-//   retention_prep   q, k of a step's rows (activation type) -> rotated, scaled fp32 rows [T, 2, H, D]
+//   retention_prep   q, k of a step's rows (activation type) -> activated, rotated, scaled fp32 rows [T, 2, H, D]
 //   retention        the recurrence over a step's items (rows of one sequence at consecutive positions + the
 //                    sequence's state slot; a decode row is an item of one row).  One workgroup of NW waves per (item,
 //                    head, 16 NW value columns): a lane keeps a quarter of one state column in registers (lane =
@@ -19,8 +20,12 @@ namespace {
 template <typename AT>
 __global__ void __launch_bounds__(256)
 retention_prep_kernel(const AT* __restrict__ proj, int ldp, int k_off, const float* __restrict__ freq, float mult,
-                      const int* __restrict__ positions, float* __restrict__ qk, int H, int D, int rd, float k_scale) {
+                      const int* __restrict__ positions, float* __restrict__ qk, int H, int D, int rd, float k_scale, int act) {
   const int t = blockIdx.x;
+  auto ld = [&](const AT* p) {
+    const float z = Elem<AT>::ld(p);
+    return act ? silu_f(z) : z;
+  };
   const float p = (float)positions[t];
   const AT* pr = proj + (size_t)t * ldp;
   float* o = qk + (size_t)t * 2 * H * D;
@@ -31,8 +36,8 @@ retention_prep_kernel(const AT* __restrict__ proj, int ldp, int k_off, const flo
     sn *= mult, cs *= mult;
     for (int h = 0; h < H; ++h) {
       const int c = h * D + i;
-      const float qu = Elem<AT>::ld(pr + c), qv = Elem<AT>::ld(pr + c + half);
-      const float ku = Elem<AT>::ld(pr + k_off + c), kv = Elem<AT>::ld(pr + k_off + c + half);
+      const float qu = ld(pr + c), qv = ld(pr + c + half);
+      const float ku = ld(pr + k_off + c), kv = ld(pr + k_off + c + half);
       o[c] = qu * cs - qv * sn;
       o[c + half] = qv * cs + qu * sn;
       o[H * D + c] = (ku * cs - kv * sn) * k_scale;
@@ -42,8 +47,8 @@ retention_prep_kernel(const AT* __restrict__ proj, int ldp, int k_off, const flo
   const int rest = D - rd;
   for (int e = threadIdx.x; e < H * rest; e += blockDim.x) {
     const int h = e / rest, c = h * D + rd + (e - h * rest);
-    o[c] = Elem<AT>::ld(pr + c);
-    o[H * D + c] = Elem<AT>::ld(pr + k_off + c) * k_scale;
+    o[c] = ld(pr + c);
+    o[H * D + c] = ld(pr + k_off + c) * k_scale;
   }
 }
 
@@ -54,7 +59,7 @@ __global__ void __launch_bounds__(64 * NW)
 retention_kernel(const float* __restrict__ qk, const AT* __restrict__ v, int ldv, const float* __restrict__ decay,
                  float* __restrict__ state, long long slot_stride, const int* __restrict__ cu,
                  const int* __restrict__ item_slot, const int* __restrict__ positions, float* __restrict__ out, int ldo,
-                 int H, int D, int Dv, int col_tiles) {
+                 int H, int D, int Dv, int col_tiles, int act) {
   constexpr int QLD = DPL + 4;   // a quarter's stride in LDS: the four quarters start in different banks
   constexpr int VT = 16 * NW;    // value columns of a workgroup
   __shared__ __attribute__((aligned(16))) float q_s[kTT][4 * QLD];
@@ -86,7 +91,8 @@ retention_kernel(const float* __restrict__ qk, const AT* __restrict__ v, int ldv
     }
     for (int e = tid; e < nt * VT; e += 64 * NW) {
       const int tt = e / VT, c = e - tt * VT;
-      v_s[tt][c] = col0 + c < Dv ? Elem<AT>::ld(v + (size_t)(t0 + tt) * ldv + (size_t)h * Dv + col0 + c) : 0.f;
+      const float z = col0 + c < Dv ? Elem<AT>::ld(v + (size_t)(t0 + tt) * ldv + (size_t)h * Dv + col0 + c) : 0.f;
+      v_s[tt][c] = act ? silu_f(z) : z;
     }
     __syncthreads();
     for (int tt = 0; tt < nt; ++tt) {
@@ -122,26 +128,26 @@ using namespace lwc;
 extern "C" int r32_retention_max_dim() { return 256; }
 
 extern "C" int r32_retention_prep(const void* proj, int ldp, int k_off, const float* freq, float mult, const int* positions,
-                                  float* qk, int T, int H, int D, int rd, float k_scale, int f32, hipStream_t s) {
+                                  float* qk, int T, int H, int D, int rd, float k_scale, int act, int f32, hipStream_t s) {
   if (T <= 0) return 0;
   if (rd % 2 != 0 || rd > D || rd < 0) return -1;
-  if (f32) retention_prep_kernel<float><<<T, 256, 0, s>>>((const float*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale);
-  else retention_prep_kernel<bf16_t><<<T, 256, 0, s>>>((const bf16_t*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale);
+  if (f32) retention_prep_kernel<float><<<T, 256, 0, s>>>((const float*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale, act);
+  else retention_prep_kernel<bf16_t><<<T, 256, 0, s>>>((const bf16_t*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale, act);
   LWC_CHECK_LAUNCH();
   return 0;
 }
 
 // qk fp32 [T, 2, H, D] from retention_prep; v rows of the activation type (leading dimension ldv), head h at columns
-// h Dv ..; state fp32 [slots, H, D, Dv]; out fp32 rows (leading dimension ldo)
+// h Dv ..; state fp32 [slots, H, D, Dv]; out fp32 rows (leading dimension ldo); act != 0: v goes through silu
 extern "C" int r32_retention(const float* qk, const void* v, int ldv, const float* decay, float* state, long long slot_stride,
                              const int* cu, const int* item_slot, const int* positions, float* out, int ldo, int items,
-                             int H, int D, int Dv, int f32, hipStream_t s) {
+                             int H, int D, int Dv, int act, int f32, hipStream_t s) {
   if (items <= 0) return 0;
   if (D < 1 || D > 256 || Dv < 1) return -1;
   const int tiles = (Dv + 15) / 16;
 #define LWC_RET2(AT, DPL, NW)                                                                                             \
   retention_kernel<AT, DPL, NW><<<dim3(H * ((tiles + NW - 1) / NW), items), 64 * NW, 0, s>>>(                            \
-      qk, (const AT*)v, ldv, decay, state, slot_stride, cu, item_slot, positions, out, ldo, H, D, Dv, (tiles + NW - 1) / NW)
+      qk, (const AT*)v, ldv, decay, state, slot_stride, cu, item_slot, positions, out, ldo, H, D, Dv, (tiles + NW - 1) / NW, act)
 #define LWC_RET(DPL, NW)       \
   if (f32) {                   \
     LWC_RET2(float, DPL, NW);  \

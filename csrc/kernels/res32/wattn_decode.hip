@@ -5,11 +5,11 @@
 // Sizes the decode kernel is built for.  vk: the caller's value pages repeat the first Dv entries of the key rows (a
 // latent that is key and value at once); only then does the wide kernel apply (it reads its values from the key rows).
 extern "C" int r32_window_attn_decode_ok(int D, int Dv, int vk) {
-  const bool small = (D == 32 || D == 64 || D == 128) && (Dv == 32 || Dv == 64 || Dv == 128);
-  return small || (vk && D == 576 && Dv == 512);
+  const bool small = (D == 32 || D == 64 || D == 128 || D == 192) && (Dv == 32 || Dv == 64 || Dv == 128);
+  return small || (vk && ((D == 576 && Dv == 512) || (D == 320 && Dv == 256)));
 }
 
-extern "C" int r32_window_attn_decode_wide_launch(const WAttnDecodeParams* p, int gx, int gy, int gz, int chunks_per_group,
+extern "C" int r32_window_attn_decode_wide_launch(const WAttnDecodeParams* p, int D, int gx, int gy, int gz, int chunks_per_group,
                                                   hipStream_t s);
 
 // out[b, h, :] = sum_s exp(m_s - M) o_s / sum_s exp(m_s - M) l_s  (splits that saw no key have l = 0)
@@ -49,10 +49,10 @@ int launch_decode_nv(const WAttnDecodeParams& p, int nv, dim3 grid, hipStream_t 
 // Splits for a decode step of B sequences whose windows hold at most max_keys keys: about 2048 waves (two per SIMD),
 // at least 64 keys each.  Measured at 64 sequences x 8 kv heads x 2048 keys of 128: 3 splits 150 us, 4 splits
 // (2048 waves) 130 us, 8 splits 155 us, 16 splits 146 us (shorter key runs per wave, larger partials to merge).
-// Wide rows (D = 576): workgroups of four or eight waves, about 512 of them, at least 128 keys each (their partials
+// Wide rows (D = 320, 576): workgroups of four or eight waves, about 512 of them, at least 128 keys each (their partials
 // are large).
 extern "C" int r32_window_attn_decode_splits(int B, int G, int Hg, int max_keys, int D) {
-  const bool wide = D > 128;
+  const bool wide = D > 192;
   const int chunks = (Hg + 15) / 16;
   const int waves = B * G * (wide && chunks > 1 ? (chunks + 1) / 2 : chunks);  // wide rows: workgroups
   int s = ((wide ? 512 : 2048) + waves - 1) / waves;
@@ -84,14 +84,15 @@ extern "C" int r32_window_attn_decode(const float* q, const void* k_cache, const
   const int Hg = H / G;
   const dim3 grid(B, G * ((Hg + 15) / 16), S);
   int rc = -1;
-  if (D == 576 && Dv == 512) {  // one wide row for all heads: a low-rank attention's cached latent + rotated part
+  if (D > 192) {  // one wide row for all heads: a low-rank attention's cached latent + rotated part
     const int chunks = (Hg + 15) / 16, nc = chunks > 1 ? 2 : 1;  // more than 16 heads: two chunks per workgroup
-    rc = r32_window_attn_decode_wide_launch(&p, B, G * ((chunks + nc - 1) / nc), S, nc, s);
+    rc = r32_window_attn_decode_wide_launch(&p, D, B, G * ((chunks + nc - 1) / nc), S, nc, s);
   } else {
     switch (D / 32) {
       case 1: rc = launch_decode_nv<1>(p, Dv / 16, grid, s); break;
       case 2: rc = launch_decode_nv<2>(p, Dv / 16, grid, s); break;
       case 4: rc = launch_decode_nv<4>(p, Dv / 16, grid, s); break;
+      case 6: rc = launch_decode_nv<6>(p, Dv / 16, grid, s); break;
     }
   }
   if (rc != 0) return rc;

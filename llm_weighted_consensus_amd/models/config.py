@@ -386,10 +386,11 @@ class RotarySpec:
 
 @dataclass(frozen=True)
 class LatentAttentionSpec:
-    """Causal softmax attention whose queries and keys / values pass through low-rank latents (``q_rank``,
-    ``kv_rank``); per head ``dim`` unrotated and ``rot_dim`` rotated query / key entries (the rotated key part is one
-    vector for all heads, pairs interleaved), values of ``vdim``; a learned sink per head in the softmax's
-    denominator; a sigmoid output gate."""
+    """Causal softmax attention whose keys / values pass through a low-rank latent (``kv_rank``), the queries too unless
+    ``q_rank`` is 0; per head ``dim`` unrotated and ``rot_dim`` rotated query / key entries (the rotated key part is one
+    vector for all heads, pairs interleaved), values of ``vdim``; a sigmoid output gate.  Whether there is a learned sink
+    per head in the softmax's denominator, and whether the gate is per entry or per head, is the design's.
+    ``kv_from``: the layer whose cached latents and rotated key parts this layer reads instead of caching its own."""
     heads: int
     dim: int
     rot_dim: int
@@ -398,6 +399,7 @@ class LatentAttentionSpec:
     kv_rank: int
     scale: float
     rot: RotarySpec
+    kv_from: Optional[int] = None
 
     kv_heads = 1   # one cached row (latent + rotated part) serves every head
 
@@ -739,8 +741,162 @@ class RerozenConfig:
         return n
 
 
+# ------------------------------------------------------------------ Gefilix
+@dataclass(frozen=True)
+class LightningSpec:
+    """Linear attention with a fixed decay per head over silu-activated q, k and v: S <- a_h S + k v^T, o = S^T q (no
+    rotation, no scale); one RMS norm over all heads' results together, a sigmoid gate per entry."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: Tuple[float, ...]
+
+    kv_heads = 0
+
+    @property
+    def nq(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def nv(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class GeluFfSpec:
+    """Ungated feed-forward W_down gelu(W_up h), erf form."""
+    ff: int
+
+
+@dataclass(frozen=True)
+class GroupedExpertsSpec:
+    """Routed experts with sigmoid scores: of ``groups`` equal runs of neighbouring experts the ``keep`` with the largest
+    sum of their two best scores are open, the ``top`` best open experts run, weighted by their scores divided by the
+    scores' sum (+ ``floor``) times ``scale``.  Every expert is a clamped gated unit without biases; ``shared_ff`` > 0: one
+    more of that width runs for every token, times the sigmoid of one logit per token."""
+    experts: int
+    top: int
+    ff: int
+    limit: float
+    scale: float = 1.0
+    groups: int = 1
+    keep: int = 1
+    shared_ff: int = 0
+    shared_limit: float = 0.0
+    alpha: float = 1.702   # fixed by the design
+    floor: float = 1e-20   # fixed by the design
+
+
+@dataclass(frozen=True)
+class GefilixLayerSpec:
+    type: str                 # "latent_attention" | "lightning"
+    mixer: object             # LatentAttentionSpec (q_rank 0) | LightningSpec
+    mlp: object               # GeluFfSpec | GroupedExpertsSpec | None
+
+
+@dataclass(frozen=True)
+class GefilixConfig:
+    """Gefilix: an fp32 residual stream normed AFTER every residual sum (x = norm(alpha x + sublayer(x)), the sublayers
+    read x itself), mixers = low-rank attention with a gate per head (a layer may read another one's latents) or lightning
+    attention, feed-forwards = ungated gelu or grouped sigmoid-routed experts with a gated shared expert; scaled
+    embedding, output weights of their own."""
+    name: str
+    vocab_size: int
+    hidden: int
+    layer_specs: Tuple[GefilixLayerSpec, ...]
+    norm_eps: float
+    alpha: float
+    embed_scale: float
+    bos_token_id: int = 1
+    eos_token_id: int = 2
+
+    architecture = "Gefilix"
+    num_experts = 0   # the engine's expert-parallel planning does not apply
+
+    @property
+    def layers(self) -> int:
+        return len(self.layer_specs)
+
+    @property
+    def heads(self) -> int:
+        return max(L.mixer.heads for L in self.layer_specs)
+
+    @property
+    def kv_heads(self) -> int:
+        return 1
+
+    @property
+    def head_dim(self) -> int:
+        return max(L.mixer.dim for L in self.layer_specs)
+
+    @classmethod
+    def from_dict(cls, c: dict, name: str = "gefilix") -> "GefilixConfig":
+        specs = []
+        for i, L in enumerate(c["layers"]):
+            m = L["mixer"]
+            if L["type"] == "latent_attention":
+                src = m.get("kv_from")
+                mixer = LatentAttentionSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]),
+                                            vdim=int(m["vdim"]), q_rank=0, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
+                                            rot=RotarySpec.from_dict(m["rot"]), kv_from=None if src is None else int(src))
+                if mixer.rot.dims != mixer.rot_dim or mixer.rot_dim % 2:
+                    raise ValueError("Gefilix: a latent attention layer rotates its whole rot_dim part (an even size)")
+                if src is not None:
+                    o = specs[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+                    if (not isinstance(o, LatentAttentionSpec) or o.kv_from is not None
+                            or (o.kv_rank, o.rot_dim, o.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot)):
+                        raise ValueError("Gefilix: kv_from names an earlier latent attention layer with latents of its own "
+                                         "and the same kv_rank, rot_dim and rotation")
+            elif L["type"] == "lightning":
+                mixer = LightningSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                      decay=tuple(float(a) for a in m["decay"]))
+                if len(mixer.decay) != mixer.heads:
+                    raise ValueError("Gefilix: one decay per lightning head")
+            else:
+                raise ValueError(f"Gefilix: unknown mixer type {L['type']!r}")
+            mlp = L.get("mlp")
+            spec = None
+            if mlp is not None:
+                if mlp.get("kind") == "dense":
+                    spec = GeluFfSpec(ff=int(mlp["ff"]))
+                elif mlp.get("kind") == "moe":
+                    r, sh, g = mlp["router"], mlp.get("shared"), mlp["router"].get("groups") or {}
+                    spec = GroupedExpertsSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(mlp["expert"]["ff"]),
+                                              limit=float(mlp["expert"]["limit"]), scale=float(r.get("scale", 1.0)),
+                                              groups=int(g.get("count", 1)), keep=int(g.get("keep", 1)),
+                                              shared_ff=int(sh["ff"]) if sh else 0, shared_limit=float(sh["limit"]) if sh else 0.0)
+                    if spec.groups < 1 or spec.experts % spec.groups or not 1 <= spec.keep <= spec.groups:
+                        raise ValueError("Gefilix: the experts form equal groups, of which at least one is kept")
+                    if not 1 <= spec.top <= spec.keep * (spec.experts // spec.groups):
+                        raise ValueError("Gefilix: router.top out of range")
+                else:
+                    raise ValueError(f"Gefilix: unknown feed-forward kind {mlp.get('kind')!r}")
+            specs.append(GefilixLayerSpec(L["type"], mixer, spec))
+        return cls(name=name, vocab_size=int(c["vocab"]), hidden=int(c["width"]), layer_specs=tuple(specs),
+                   norm_eps=float(c["norm"]["eps"]), alpha=float(c["postln_alpha"]), embed_scale=float(c["embedding"]["scale"]))
+
+    def params(self) -> int:
+        d = self.hidden
+        n = 2 * self.vocab_size * d + d
+        for L in self.layer_specs:
+            m, e = L.mixer, L.mlp
+            n += d + d * m.nv
+            if L.type == "latent_attention":
+                n += d * (m.nq + m.heads) + m.kv_rank * m.heads * (m.dim + m.vdim)
+                if m.kv_from is None:
+                    n += d * (m.kv_rank + m.rot_dim) + m.kv_rank
+            else:
+                n += d * (2 * m.nq + 2 * m.nv) + m.nv
+            if isinstance(e, GeluFfSpec):
+                n += d + 2 * d * e.ff
+            elif e is not None:
+                n += d + (e.experts * e.ff + e.shared_ff) * 3 * d + e.experts * d + (d if e.shared_ff else 0)
+        return n
+
+
 # config.json "architecture" -> config class of the layer-list decoders
-ARCHITECTURES = {"Madipel": MadipelConfig, "Merudra": MerudraConfig, "Limatar": LimatarConfig, "Rerozen": RerozenConfig}
+ARCHITECTURES = {"Madipel": MadipelConfig, "Merudra": MerudraConfig, "Limatar": LimatarConfig, "Rerozen": RerozenConfig,
+                 "Gefilix": GefilixConfig}
 
 
 def load_model_config(model_dir) -> object:

@@ -12,8 +12,8 @@ from typing import Optional
 
 import torch
 
-from .config import (DECODERS, LimatarConfig, MadipelConfig, MerudraConfig, RerozenConfig, decoder_config,
-                     load_model_config)
+from .config import (ARCHITECTURES, DECODERS, GefilixConfig, LimatarConfig, MadipelConfig, MerudraConfig, RerozenConfig,
+                     decoder_config, load_model_config)
 
 DTYPES = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32, "fp32": torch.float32}
 
@@ -42,6 +42,10 @@ def model_class(cfg):
         from .rerozen import RerozenModel
 
         return RerozenModel
+    if isinstance(cfg, GefilixConfig):
+        from .gefilix import GefilixModel
+
+        return GefilixModel
     if getattr(cfg, "num_experts", 0):
         from .mixtral import MixtralModel
 
@@ -57,7 +61,7 @@ def load_model(model_dir: str, device="cuda", dtype=torch.bfloat16, max_position
     instead of the folder's."""
     cfg = load_model_config(model_dir)
     cls = model_class(cfg)
-    if dtype != torch.bfloat16 and not isinstance(cfg, (MadipelConfig, MerudraConfig, LimatarConfig, RerozenConfig)):
+    if dtype != torch.bfloat16 and not isinstance(cfg, tuple(ARCHITECTURES.values())):
         raise ValueError(f"{cfg.name}: this decoder runs in bfloat16 only")
     path = None if random_seed is not None else str(Path(model_dir))
     return cls(cfg, device=device, dtype=dtype, seed=random_seed or 0, weights_path=path, max_position=max_position)

@@ -195,11 +195,11 @@ def head_norm_gate(o: torch.Tensor, out: torch.Tensor, H: int, eps: float, w: Op
 
 
 def embed_rows(table: torch.Tensor, tokens: torch.Tensor, out: Optional[torch.Tensor] = None,
-               scale: float = 1.0) -> torch.Tensor:
-    """x[t] = table[tokens[t]] * scale as fp32."""
+               scale: float = 1.0, cast: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x[t] = table[tokens[t]] * scale as fp32; ``cast`` (bf16 [T, d]) also receives the rows."""
     if out is None:
         out = torch.empty(tokens.numel(), table.shape[1], dtype=torch.float32, device=table.device)
-    kernels().embed_rows(table, tokens, out, float(scale))
+    kernels().embed_rows(table, tokens, out, float(scale), cast)
     return out
 
 
@@ -255,25 +255,51 @@ def stack_mix(X: torch.Tensor, coef: torch.Tensor, n: int, out: torch.Tensor) ->
 
 
 def router(z: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int,
-           bias: Optional[torch.Tensor] = None, renorm: bool = False):
-    """Softmax router over all outputs of ``z`` (fp32 [T, NE]) + ``bias``; the ``top`` largest of softmax + correction
-    are chosen, weighted by their softmax (``renorm``: divided by the chosen ones' sum, which is the softmax over the
-    chosen logits only).  Outputs >= ``experts`` are identity experts.  Returns
+           bias: Optional[torch.Tensor] = None, renorm: bool = False, scores: str = "softmax", floor: float = 0.0,
+           scale: float = 1.0, groups: int = 1, keep: int = 1):
+    """Router over all outputs of ``z`` (fp32 [T, NE], a column slice is fine) + ``bias``.  ``scores``: "softmax" over all
+    outputs, or "sigmoid" of each.  The ``top`` largest of score + correction are chosen, weighted by their scores
+    (``renorm``: divided by the chosen ones' sum + ``floor``; for a softmax with floor 0 that is the softmax over the
+    chosen logits only) times ``scale``.  ``groups`` > 1: the outputs form that many equal runs of neighbours, and only
+    outputs of the ``keep`` runs with the largest sum of their two best scores can be chosen.
+    Outputs >= ``experts`` are identity experts.  Returns
     (ids [T, top], w [T, top], row_off [experts + 1], src [T top], row_expert [T top], inv [T top]): expert-major
     row r holds token src[r] for expert row_expert[r]; choice (t, j) is row inv[t top + j], -1 for an identity."""
-    return tuple(kernels().router(z, correction, int(experts), int(top), bias, bool(renorm)))
+    return tuple(kernels().router(z, correction, int(experts), int(top), bias, bool(renorm), scores == "sigmoid", float(floor),
+                                  float(scale), int(groups), int(keep)))
 
 
 def expert_rows(h: torch.Tensor, src: torch.Tensor, row_expert: torch.Tensor, row_off: torch.Tensor, w_gu: torch.Tensor,
-                w_down: torch.Tensor) -> torch.Tensor:
-    """Y[r] = W_down[e] (silu(W_gate[e] h) * (W_up[e] h)) for every expert-major row r (fp32 sums, any sizes)."""
-    return kernels().expert_rows(h, src, row_expert, row_off, w_gu, w_down)
+                w_down: torch.Tensor, mode: str = "silu", alpha: float = 1.0, limit: float = 0.0) -> torch.Tensor:
+    """Y[r] = W_down[e] act(W_gate[e] h, W_up[e] h) for every expert-major row r (fp32 sums, any sizes); ``mode``,
+    ``alpha``, ``limit``: the gated unit, as in :func:`glu`."""
+    return kernels().expert_rows(h, src, row_expert, row_off, w_gu, w_down, mode == "clamped", float(alpha), float(limit))
 
 
 def moe_combine(Y: torch.Tensor, inv: torch.Tensor, w: torch.Tensor, h: torch.Tensor,
-                add: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """fp32 [T, d]: sum_j w[t, j] * (Y[inv[t, j]] if inv >= 0 else h[t]) (+ ``add[t]``: a shared expert's rows)."""
-    return kernels().moe_combine(Y, inv, w, h, add)
+                add: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 [T, d]: sum_j w[t, j] * (Y[inv[t, j]] if inv >= 0 else h[t]) (+ ``add[t]``: a shared expert's rows, times
+    sigmoid(``gate[t]``) with ``gate`` fp32 [T])."""
+    return kernels().moe_combine(Y, inv, w, h, add, gate)
+
+
+def post_norm(x: torch.Tensor, y: torch.Tensor, alpha: float, w: torch.Tensor, eps: float,
+              cast: Optional[torch.Tensor] = None) -> None:
+    """x (fp32) <- v / rms(v) * w with v = alpha x + y, in place: a sublayer whose norm comes after the residual sum.
+    ``cast`` (bf16 [T, d]) also receives the new x."""
+    kernels().post_norm(x, y, float(alpha), w, float(eps), cast)
+
+
+def post_norm_experts(x: torch.Tensor, Y: torch.Tensor, inv: torch.Tensor, wts: torch.Tensor, h: torch.Tensor, alpha: float,
+                      w: torch.Tensor, eps: float, shared: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                      cast: Optional[torch.Tensor] = None) -> None:
+    """:func:`post_norm` of the routed sum :func:`moe_combine` (``shared`` rows times sigmoid(``gate``)), in one pass: the
+    sum stays in registers (rows of a width that is no multiple of four, or above 8192: two passes)."""
+    K = kernels()
+    if K.post_norm_experts_ok(x.shape[1]):
+        K.post_norm_experts(x, Y, inv, wts, shared, gate, float(alpha), w, float(eps), cast)
+    else:
+        K.post_norm(x, K.moe_combine(Y, inv, wts, h, shared, gate), float(alpha), w, float(eps), cast)
 
 
 # ------------------------------------------------------------------ rotations, low-rank attention, retention, gated units
@@ -299,14 +325,14 @@ def rope_frequencies(dims: int, base: float, scaling: Optional[dict] = None, dev
     return f.to(torch.float32).to(device), m
 
 
-def latent_kv_write(proj: torch.Tensor, Cq: int, C: int, R: int, wq: torch.Tensor, wc: torch.Tensor, freq: torch.Tensor,
+def latent_kv_write(proj: torch.Tensor, Cq: int, C: int, R: int, wq: Optional[torch.Tensor], wc: torch.Tensor, freq: torch.Tensor,
                     mult: float, positions: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
-                    eps: float, cq: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    eps: float, cq: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """Cache side of a low-rank attention layer.  ``proj`` rows = [dq (Cq) | c (C) | key part to rotate (R) | ...]:
-    returns cq = dq / rms(dq) * wq ([T, Cq], proj's dtype); writes per token ONE key row [c / rms(c) * wc | rotated
+    returns cq = dq / rms(dq) * wq ([T, Cq], proj's dtype; ``Cq`` 0: queries without a latent, returns None); writes per token ONE key row [c / rms(c) * wc | rotated
     part * mult | zeros] and the same normalised c as its value row into the paged cache at ``slots`` (-1: no write).
     Rotation: entries (2i, 2i + 1) by the angle position * freq[i]."""
-    if cq is None:
+    if cq is None and Cq:
         cq = torch.empty(proj.shape[0], Cq, dtype=proj.dtype, device=proj.device)
     kernels().latent_kv_write(proj, int(Cq), int(C), int(R), wq, wc, freq, float(mult), positions, slots, cq, k_cache,
                               v_cache, float(eps))
@@ -323,6 +349,13 @@ def latent_q_rows(q: torch.Tensor, D: int, R: int, qn: Optional[torch.Tensor], f
     return out
 
 
+def head_gate_rows(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out[t, h Dv + i] = o[t, h, i] * sigmoid(gate[t, h]); ``o`` [T, H, Dv] of any row and head strides (a batched product
+    as it lies, padded heads), ``gate`` [T, H] (a column slice is fine)."""
+    kernels().head_gate_rows(o, gate, out)
+    return out
+
+
 def latent_expand_write(kv: torch.Tensor, lat: torch.Tensor, rot_off: int, R: int, slots: torch.Tensor, k_cache: torch.Tensor,
                         v_cache: torch.Tensor, H: int, D: int, Dv: int) -> None:
     """Keys and values up-projected from cached latents, written as pages of their own: ``kv`` [N, H D + H Dv], ``lat``
@@ -333,17 +366,27 @@ def latent_expand_write(kv: torch.Tensor, lat: torch.Tensor, rot_off: int, R: in
 
 def retention(proj: torch.Tensor, k_off: int, v: torch.Tensor, freq: torch.Tensor, mult: float, rot_dims: int,
               decay: torch.Tensor, state: torch.Tensor, items: StepItems, H: int,
-              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+              out: Optional[torch.Tensor] = None, k_scale: Optional[float] = None, act: bool = False) -> torch.Tensor:
     """Retention over a step's items: per head S <- a_h S + k v^T, o = S^T q (no softmax, no denominator).  q (columns
     0 ..) and k (columns ``k_off`` ..) of ``proj`` are rotated on their first ``rot_dims`` entries (entry i with
-    i + rot_dims / 2, angle position * freq[i]); k is then multiplied by D^-1/2.  ``v`` [T, H Dv] (a column slice of
+    i + rot_dims / 2, angle position * freq[i]); k is then multiplied by ``k_scale`` (D^-1/2 when None).  ``act``: q, k
+    and v go through silu first.  ``v`` [T, H Dv] (a column slice of
     ``proj`` is fine), ``state`` fp32 [slots, H, D, Dv] (read unless the item starts at position 0, written back).
     Returns o fp32 [T, H Dv]."""
     if out is None:
         out = torch.empty(proj.shape[0], H * state.shape[3], dtype=torch.float32, device=proj.device)
     kernels().retention(proj, int(k_off), v, freq, float(mult), int(rot_dims), decay, state, items.cu, items.slots,
-                        items.positions, out, int(H))
+                        items.positions, out, int(H), state.shape[2] ** -0.5 if k_scale is None else float(k_scale), bool(act))
     return out
+
+
+def lightning(proj: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, items: StepItems, H: int,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Lightning attention over a step's items: ``proj`` rows = [q (H D) | k (H D) | v (H Dv) | ...], each through silu;
+    per head S <- a_h S + k v^T, o = S^T q (no rotation, no scale).  ``state`` fp32 [slots, H, D, Dv] (read unless the
+    item starts at position 0, written back).  Returns o fp32 [T, H Dv]."""
+    nq, nv = H * state.shape[2], H * state.shape[3]
+    return retention(proj, nq, proj[:, 2 * nq:2 * nq + nv], decay[:0], 1.0, 0, decay, state, items, H, out=out, k_scale=1.0, act=True)
 
 
 def glu(gu: torch.Tensor, out: Optional[torch.Tensor] = None, mode: str = "silu", alpha: float = 1.0,
