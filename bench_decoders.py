@@ -3,7 +3,7 @@
 
     python bench.py --compare-decoders [--sizes small,8b-layer] [--compare-layers 4]
 
-Designs: ``madipel``, ``llama``, ``merudra``, ``mixtral``, ``limatar``, ``rerozen`` (``--designs merudra,mixtral`` puts Merudra
+Designs: ``madipel``, ``llama``, ``merudra``, ``mixtral``, ``limatar``, ``rerozen``, ``gefilix`` (``--designs merudra,mixtral`` puts Merudra
 beside the closest existing decoder, the routed-experts Mixtral: 8 experts, 2 per token, the same active feed-forward
 width; Merudra's layers alternate attention and gated delta rule mixers and add 2 identity experts.
 ``--designs limatar,merudra`` puts Limatar beside Merudra, the closest decoder with paged attention AND recurrent
@@ -11,7 +11,11 @@ layers over an fp32 stream: Limatar's layers alternate low-rank attention (laten
 retention, routed experts with a shared expert and the clamped dense unit).
 ``--designs rerozen,merudra`` puts Rerozen beside Merudra, the closest decoder (input convolutions in front of every
 sublayer, paged attention and gated delta rule layers over an fp32 stream): every Rerozen layer runs a chunked rotary
-attention AND a half-size channel-decay linear attention side by side, and a dense gelu feed-forward).
+attention AND a half-size channel-decay linear attention side by side, and a dense gelu feed-forward.
+``--designs gefilix,limatar`` puts Gefilix beside Limatar, the closest decoder (low-rank attention over the same cached
+rows and a fixed-decay recurrence over an fp32 stream): Gefilix's layers alternate low-rank attention, of which every
+second one reads the latents of the one before, and lightning attention, grouped sigmoid-routed clamped experts with a
+gated shared expert and the dense gelu unit).
 
 For each size a Madipel model (parallel layers, windowed attention with distance bias, xIELU feed-forward, fp32
 residual) and the closest existing decoder (Llama: sequential layers, causal GQA attention with RoPE, SwiGLU) are
@@ -127,6 +131,34 @@ def _rerozen(size: dict, layers: int, device, seed: int, pattern: str = "p2", ch
     return RerozenModel(cfg, device=device, seed=seed)
 
 
+def _gefilix(size: dict, layers: int, device, seed: int, experts: int = 8, top: int = 2, pattern: str = "lr"):
+    """Low-rank attention and lightning layers alternating (``pattern``: l / r per layer, repeated; a / d and p / 2 of the
+    other designs' patterns mean the same), sizes as in ``_limatar``; every second attention layer reads the latents of the
+    one before.  Feed-forwards alternate in pairs between routed experts (two groups of which one is open, inner width
+    ffn / top, a shared expert of ffn / 8) and the dense gelu unit of 1.5 ffn (two matrices: equal parameters)."""
+    from llm_weighted_consensus_amd.models.config import GefilixConfig
+    from llm_weighted_consensus_amd.models.gefilix import GefilixModel
+
+    H, D, d = size["heads"], size["head_dim"], size["width"]
+    moe = {"kind": "moe", "expert": {"ff": size["ffn"] // top, "limit": 7.0}, "shared": {"ff": size["ffn"] // 8, "limit": 7.0},
+           "router": {"experts": experts, "top": top, "groups": {"count": 2, "keep": 1}, "scale": 2.5}}
+    dense = {"kind": "dense", "ff": 3 * size["ffn"] // 2}
+    lat = {"heads": H, "dim": D, "rot_dim": D // 2, "vdim": D, "kv_rank": 4 * D, "scale": (D + D // 2) ** -0.5,
+           "rot": {"base": 10000.0, "dims": D // 2}}
+    lin = {"heads": H, "dim": D, "vdim": D, "decay": [1.0 - 2.0 ** (-4 - 4 * h / max(H - 1, 1)) for h in range(H)]}
+    specs, own = [], None
+    for i in range(layers):
+        mlp = moe if (i // 2 + i) % 2 == 0 else dense
+        if pattern[i % len(pattern)] in "lap":
+            specs.append({"type": "latent_attention", "mixer": lat if own is None else dict(lat, kv_from=own), "mlp": mlp})
+            own = i if own is None else None
+        else:
+            specs.append({"type": "lightning", "mixer": lin, "mlp": mlp})
+    cfg = GefilixConfig.from_dict({"architecture": "Gefilix", "embedding": {"scale": 1.0}, "layers": specs, "norm": {"eps": 1e-6},
+                                   "postln_alpha": 2.0, "vocab": size["vocab"], "width": d}, name="gefilix-bench")
+    return GefilixModel(cfg, device=device, seed=seed)
+
+
 def _mixtral(size: dict, layers: int, max_pos: int, device, seed: int, experts: int = 8, top: int = 2):
     from llm_weighted_consensus_amd.models.config import DecoderConfig
     from llm_weighted_consensus_amd.models.mixtral import MixtralModel
@@ -189,6 +221,8 @@ def run(sizes: str = "small,8b-layer", layers: int = 4, prompt_len: int = 2048, 
                 model = _merudra(size, layers, dev, 3, pattern="".join({"l": "a", "r": "d", "p": "a", "2": "d"}.get(c, c) for c in pattern))
             elif design == "rerozen":
                 model = _rerozen(size, layers, dev, 3, pattern=pattern)
+            elif design == "gefilix":
+                model = _gefilix(size, layers, dev, 3, pattern=pattern)
             elif design == "limatar":
                 model = _limatar(size, layers, dev, 3, pattern=pattern)
             elif design == "mixtral":
@@ -204,7 +238,8 @@ def run(sizes: str = "small,8b-layer", layers: int = 4, prompt_len: int = 2048, 
                     **{k: round(v, 3) for k, v in r.items()}, "dtype": "bf16", "data": "synthetic"}
             print(json.dumps(line), flush=True)
             summary.setdefault(name, {})[design] = r
-    for a, b in (("madipel", "llama"), ("merudra", "mixtral"), ("merudra", "madipel"), ("limatar", "merudra"), ("rerozen", "merudra")):
+    for a, b in (("madipel", "llama"), ("merudra", "mixtral"), ("merudra", "madipel"), ("limatar", "merudra"), ("rerozen", "merudra"),
+                 ("gefilix", "limatar")):
         out = {}
         for name, d in summary.items():
             if a in d and b in d:
