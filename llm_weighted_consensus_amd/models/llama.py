@@ -446,7 +446,8 @@ class LlamaModel:
         none = {"attn": False, "mlp": False, "final": False, "qkv_bn": 192, "o": "plain", "down": "plain"}
         # below 256 rows the chain's 256-row tiles run mostly empty and the weight-streaming cores win every
         # projection: not timed (a serving engine meets many such buckets)
-        if (cfg.hidden + 255) // 256 > 16 or M < 256:
+        # (the folded consumers and producers are gemm4w's epilogues: nothing to time while it is switched off)
+        if (cfg.hidden + 255) // 256 > 16 or M < 256 or not ops.GEMM4W:
             self.chain_m[M] = none
             return
         if self.chain is None:  # once, for every decode bucket (captured graphs keep these addresses)

@@ -427,6 +427,12 @@ def skinny_ok(M: int, N: int, K: int, swiglu: bool = False) -> bool:
     return 0 < M <= 64 and K % 2048 == 0 and N % (64 if swiglu else 16) == 0
 
 
+# gemm4w is switched off: its main loop was rewritten and the first headline run of the new build ended in a GPU fault
+# whose cause is not known.  The planners leave its backends out, a direct call raises, its tests are skipped
+GEMM4W = False
+GEMM4W_OFF = "gemm4w is switched off (a GPU fault of unknown cause in the first headline run with its rewritten main loop)"
+
+
 def gemm4w(A: torch.Tensor, W: torch.Tensor, residual: Optional[torch.Tensor] = None,
            out: Optional[torch.Tensor] = None, swiglu: bool = False, bias: Optional[torch.Tensor] = None,
            gelu: bool = False, bn: int = 256, chain: "Optional[NormChain]" = None, var: int = 0,
@@ -447,6 +453,8 @@ def gemm4w(A: torch.Tensor, W: torch.Tensor, residual: Optional[torch.Tensor] = 
     workgroup waits on one that has not started).  For shapes whose tile count leaves CUs idle (the serving
     path's mid-size row counts: :func:`split_plan`) and a ragged last round (``split_from`` = the whole
     rounds).  The workspace is this module's, sized before graph capture (:func:`split_workspace`)."""
+    if not GEMM4W:
+        raise RuntimeError(GEMM4W_OFF)
     N = W.shape[0] // 2 if swiglu else W.shape[0]
     if out is None:
         out = torch.empty(A.shape[0], N, dtype=torch.bfloat16, device=A.device)

@@ -16,6 +16,8 @@ Backends computing ``A . W^T`` for the dense projections:
   serving path's mid-size row counts: o / down at M = 2048 are 128 tiles for 256 CUs) run every tile as 2-4
   K-range units, a ragged last round (lm_head) splits only that round's tiles.
 
+The gemm4w backends (``g4*``) are left out of every choice while ``ops.GEMM4W`` is off.
+
 The hand-written cores also fuse the SwiGLU of the gate|up projection, or the residual add of the o /
 down projections (:func:`linear_add_`), into their epilogue.  None wins everywhere
 (``profiles/gemm4w.md``), so the choice is made per (M, N, K, epilogue) by timing every applicable
@@ -32,7 +34,7 @@ from typing import Dict, Optional, Tuple
 import torch
 import torch.nn.functional as F
 
-from . import gemm4w, gemm8p, silu_mul, skinny_gemm, skinny_ok, split_plan
+from . import GEMM4W, gemm4w, gemm8p, silu_mul, skinny_gemm, skinny_ok, split_plan
 
 MODE = os.environ.get("LWC_GEMM", "auto")
 BACKENDS = ("blas", "g8", "g4", "g4n192", "g4p", "gv", "g4s")
@@ -41,6 +43,9 @@ BACKENDS = ("blas", "g8", "g4", "g4n192", "g4p", "gv", "g4s")
 # engine.LLMEngine._step_ab, which sees the step's clock and cache state)
 OWN_MARGIN = float(os.environ.get("LWC_GEMM_OWN_MARGIN", "0"))
 EXCLUDE = {b for b in os.environ.get("LWC_GEMM_NO", "").split(",") if b}
+G4 = ("g4", "g4n192", "g4p", "g4s")   # the gemm4w backends: left out of every choice while ops.GEMM4W is off
+if not GEMM4W:
+    EXCLUDE.update(G4)
 # LWC_GEMM_SKINNY=0 leaves the skinny decode GEMM out of the timing (A/B knob)
 SKINNY = os.environ.get("LWC_GEMM_SKINNY", "1") != "0"
 _CHOICE: Dict[Tuple[int, int, int, str], str] = {}
@@ -151,10 +156,10 @@ def linear_bias(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, gelu: bool = 
     # gemm4w runs such an A as row blocks
     ok = _g8_ok(N, K, epi) and x.stride(1) == 1 and x.is_cuda
     small_a = M * x.stride(0) * 2 < (1 << 31)
-    runs = {"g4": lambda: gemm4w(x, w, bias=b, gelu=gelu),
-            "g4p": lambda: gemm4w(x, w, bias=b, gelu=gelu, var=64),
-            "blas": ((lambda: torch._addmm_activation(b, x, w.t(), use_gelu=True)) if gelu
+    runs = {"blas": ((lambda: torch._addmm_activation(b, x, w.t(), use_gelu=True)) if gelu
                      else (lambda: F.linear(x, w, b)))}
+    if GEMM4W:
+        runs.update({"g4": lambda: gemm4w(x, w, bias=b, gelu=gelu), "g4p": lambda: gemm4w(x, w, bias=b, gelu=gelu, var=64)})
     if small_a:
         runs["g8"] = lambda: gemm8p(x, w, bias=b, gelu=gelu, ws=ws)
     if c is None:
@@ -163,7 +168,7 @@ def linear_bias(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, gelu: bool = 
         else:
             t = {name: _time(fn, iters=2, rounds=3) for name, fn in runs.items()}
             TIMINGS[key] = t
-            own = min((n for n in ("g8", "g4", "g4p") if n in t), key=lambda n: t[n])
+            own = min((n for n in t if n != "blas"), key=lambda n: t[n], default="blas")
             c = own if t[own] <= t["blas"] * (1 + OWN_MARGIN) else "blas"
         _CHOICE[key] = c
     # (a choice made for the token bucket at a smaller A may name gemm8p, which a 2 GiB A cannot take)
@@ -183,8 +188,9 @@ def linear_residual_(x: torch.Tensor, w: torch.Tensor, acc: torch.Tensor, ws=Non
     small_a = M * x.stride(0) * 2 < (1 << 31)
 
     def runs_on(a):
-        r = {"g4": lambda: gemm4w(x, w, residual=a, out=a), "g4p": lambda: gemm4w(x, w, residual=a, out=a, var=64),
-             "blas": lambda: a.addmm_(x, w.t())}
+        r = {"blas": lambda: a.addmm_(x, w.t())}
+        if GEMM4W:
+            r.update({"g4": lambda: gemm4w(x, w, residual=a, out=a), "g4p": lambda: gemm4w(x, w, residual=a, out=a, var=64)})
         if small_a:
             r["g8"] = lambda: gemm8p(x, w, residual=a, out=a, ws=ws)
         return r
@@ -197,7 +203,7 @@ def linear_residual_(x: torch.Tensor, w: torch.Tensor, acc: torch.Tensor, ws=Non
             t = {name: _time(fn, iters=2, rounds=3) for name, fn in runs_on(scratch).items()}
             del scratch
             TIMINGS[key] = t
-            own = min((n for n in ("g8", "g4", "g4p") if n in t), key=lambda n: t[n])
+            own = min((n for n in t if n != "blas"), key=lambda n: t[n], default="blas")
             c = own if t[own] <= t["blas"] * (1 + OWN_MARGIN) else "blas"
         _CHOICE[key] = c
     runs = runs_on(acc)

@@ -10,6 +10,16 @@ from tests import torch_ref as ref
 pytestmark = pytest.mark.gpu
 
 
+def _gemm4w_on():
+    from llm_weighted_consensus_amd import ops
+
+    return ops.GEMM4W
+
+
+needs_gemm4w = pytest.mark.skipif(not _gemm4w_on(), reason="gemm4w is switched off: a GPU fault of unknown cause in the first headline "
+                                                           "run with its rewritten main loop")
+
+
 def _bf(*shape, dev, scale=1.0, g=None):
     return (torch.randn(*shape, device=dev, generator=g) * scale).to(torch.bfloat16)
 
@@ -766,6 +776,8 @@ def test_linear_add_inplace(gpu, backend, M, N, K):
     the first call's result."""
     from llm_weighted_consensus_amd.ops import gemm_plan
 
+    if backend in gemm_plan.G4 and not _gemm4w_on():
+        pytest.skip("gemm4w is switched off: a GPU fault of unknown cause in the first headline run with its rewritten main loop")
     torch.manual_seed(M + K)
     A = torch.randn(M, K, device=gpu).to(torch.bfloat16)
     W = (torch.randn(N, K, device=gpu) / K ** 0.5).to(torch.bfloat16)
@@ -1279,6 +1291,7 @@ def test_gemm8p_bias_gelu_epilogue(gpu, M, N, K, gelu):
     _close(gemm_plan.linear_bias(A, W, b, gelu=gelu), ref, 3e-2, 1e-2)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("var", [32, 64])
 @pytest.mark.parametrize("bn", [256, 192])
 @pytest.mark.parametrize("M,N,K,epi", [(300, 520, 64, "plain"), (4096, 6144, 4096, "plain"), (513, 1000, 128, "res"),
@@ -1326,6 +1339,7 @@ def test_gemm4w(gpu, M, N, K, epi, bn, var):
             _close(out, want, 3e-2, 1e-2)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("var", [32, 64])
 @pytest.mark.parametrize("M,N,K,epi,bn,P", [(300, 4096, 256, "plain", 256, 1), (4096 + 37, 6144, 512, "plain", 192, 16),
                                            (1000, 1536, 320, "swiglu", 256, 3), (257, 128256 // 16, 128, "plain", 256, 2),
@@ -1357,6 +1371,7 @@ def test_gemm4w_rowscale(gpu, M, N, K, epi, bn, P, var):
             _close(ops.gemm4w(A, W, bn=bn, chain=chain, var=var), ref, 3e-2, 1e-2)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("var", [32, 64])
 @pytest.mark.parametrize("M,N,K", [(4096, 4096, 256), (300, 4096, 512), (1000, 1024, 128), (4096 + 37, 4096, 64)])
 def test_gemm4w_residual_rowsum(gpu, M, N, K, var):
@@ -1460,6 +1475,7 @@ def test_skinny_gemm_swiglu_matches_fp32(gpu, M, N, K):
     assert out.shape == (M, F)
     _close(out, torch.nn.functional.silu(ref[:, :F]) * ref[:, F:], 3e-2, 1e-2)
 
+@needs_gemm4w
 def test_gemm4w_row_blocks_past_2gib(gpu):
     """gemm4w addresses A through one 32-bit buffer range; ops.gemm4w runs an A of 2 GiB or more (the encoders'
     FFN2 input at config 2's 0.5 M tokens is 3 GiB) as row blocks: rows on both sides of the block boundary and
@@ -1483,6 +1499,7 @@ def test_gemm4w_row_blocks_past_2gib(gpu):
         _close(R[r0:r1], ref + R0[r0:r1].float(), 3e-2, 1e-2)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("splits", [2, 3, 4])
 @pytest.mark.parametrize("M,N,K,epi,split_from", [(2048, 4096, 4096, "res", 0), (700, 2048, 1024, "swiglu", 0),
                                                   (1000, 128256 // 16, 512, "plain", 64), (300, 6144, 512, "plain", 0),
@@ -1514,6 +1531,7 @@ def test_gemm4w_split_k(gpu, M, N, K, epi, split_from, splits):
     assert int(cnt.abs().sum()) == 0  # every tile's counters were reset by its last arriver
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("M,N,K,splits", [(2560, 4096, 1024, 7), (2304, 4096, 1792, 3), (2560, 4096, 3584, 6)])
 def test_gemm4w_split_k_uneven(gpu, M, N, K, splits):
     """Split-K with S not dividing the K tile count (units of K tile pairs [s H / S, (s + 1) H / S), H = K / 128)
@@ -1534,6 +1552,7 @@ def test_gemm4w_split_k_uneven(gpu, M, N, K, splits):
     assert int(cnt.abs().sum()) == 0
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("splits", [2, 3, 4])
 def test_gemm4w_split_k_norm_chain(gpu, splits):
     """Split-K with the folded-RMSNorm epilogues: a row-scaled consumer (RS 1) and a residual producer that
@@ -1558,6 +1577,7 @@ def test_gemm4w_split_k_norm_chain(gpu, splits):
     assert torch.allclose(chain.ss[:N // 256, :M], parts, rtol=1e-5, atol=1e-4)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("var", [32, 64])
 def test_gemm4w_gelu_epilogue_values(gpu, var):
     """The GELU epilogue's math alone: W = identity, so the output is gelu(A + b) of the operand's own bf16
@@ -1573,6 +1593,7 @@ def test_gemm4w_gelu_epilogue_values(gpu, var):
     _close(y, torch.nn.functional.gelu(x.float()), 1e-3, 8e-3)
 
 
+@needs_gemm4w
 @pytest.mark.parametrize("var", [32, 64])
 def test_gemm4w_operand_past_2gib_one_launch(gpu, var):
     """A of more than 2 GiB in one launch (the kernel's A buffer resource spans one tile's rows): the first

@@ -312,6 +312,8 @@ def test_folded_norm_chain_matches_unfolded(tiny, gpu, qkv_bn):
     from llm_weighted_consensus_amd import ops
     from llm_weighted_consensus_amd.models.llama import KVCache
 
+    if not ops.GEMM4W:
+        pytest.skip("gemm4w is switched off: a GPU fault of unknown cause in the first headline run with its rewritten main loop")
     m = tiny
     assert m.norm_folded and bool((m.layers[0].attn_norm == 1).all())
     cache = KVCache(m.cfg, 64, 16, gpu)

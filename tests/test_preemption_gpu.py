@@ -22,10 +22,10 @@ def test_kv_oversubscription_swaps_and_matches_uninterrupted(tiny, gpu):
     from llm_weighted_consensus_amd.ops import gemm_plan
 
     # a batch-composition-invariant forward, so the two runs can be compared token for token: every GEMM
-    # on gemm4w (a row's result does not depend on the other rows), split-K 1 and the wave-per-item
-    # decode kernel for every batch, no cascade tiles
+    # on gemm8p (every call here is one 256-row tile high, so a row's result does not depend on the other
+    # rows), split-K 1 and the wave-per-item decode kernel for every batch, no cascade tiles
     old_mode, old_min = gemm_plan.MODE, ops.set_decode_wave_min_items(0)
-    gemm_plan.MODE = "g4"
+    gemm_plan.MODE = "g8"
     try:
         tok = ByteTokenizer(tiny.cfg.vocab_size)
         prompts = [tok.encode(f"request {i}: " + "abcdefgh"[i] * (20 + 3 * i)) for i in range(6)]
