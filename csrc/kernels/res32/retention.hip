@@ -17,14 +17,14 @@
 namespace lwc {
 namespace {
 
-template <typename AT>
+template <typename AT, bool ACT>
 __global__ void __launch_bounds__(256)
 retention_prep_kernel(const AT* __restrict__ proj, int ldp, int k_off, const float* __restrict__ freq, float mult,
-                      const int* __restrict__ positions, float* __restrict__ qk, int H, int D, int rd, float k_scale, int act) {
+                      const int* __restrict__ positions, float* __restrict__ qk, int H, int D, int rd, float k_scale) {
   const int t = blockIdx.x;
-  auto ld = [&](const AT* p) {
+  auto ld = [](const AT* p) {
     const float z = Elem<AT>::ld(p);
-    return act ? silu_f(z) : z;
+    return ACT ? silu_f(z) : z;
   };
   const float p = (float)positions[t];
   const AT* pr = proj + (size_t)t * ldp;
@@ -49,6 +49,22 @@ retention_prep_kernel(const AT* __restrict__ proj, int ldp, int k_off, const flo
     const int h = e / rest, c = h * D + rd + (e - h * rest);
     o[c] = ld(pr + c);
     o[H * D + c] = ld(pr + k_off + c) * k_scale;
+  }
+}
+
+// Activated rows without a rotation (k_scale on the second half), four entries per thread: n = H D a multiple of four
+template <typename AT>
+__global__ void __launch_bounds__(256)
+lightning_prep_vec_kernel(const AT* __restrict__ proj, int ldp, int k_off, float* __restrict__ qk, int n, float k_scale) {
+  const int t = blockIdx.x;
+  const AT* pr = proj + (size_t)t * ldp;
+  float* o = qk + (size_t)t * 2 * n;
+#pragma unroll 4
+  for (int e = threadIdx.x * 4; e < 2 * n; e += 1024) {
+    const bool isk = e >= n;
+    const float4v z = Vec4<AT>::ld(pr + (isk ? k_off + e - n : e));
+    const float4v a = float4v{silu_f(z[0]), silu_f(z[1]), silu_f(z[2]), silu_f(z[3])};
+    Vec4<float>::st(o + e, isk ? a * k_scale : a);
   }
 }
 
@@ -131,8 +147,20 @@ extern "C" int r32_retention_prep(const void* proj, int ldp, int k_off, const fl
                                   float* qk, int T, int H, int D, int rd, float k_scale, int act, int f32, hipStream_t s) {
   if (T <= 0) return 0;
   if (rd % 2 != 0 || rd > D || rd < 0) return -1;
-  if (f32) retention_prep_kernel<float><<<T, 256, 0, s>>>((const float*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale, act);
-  else retention_prep_kernel<bf16_t><<<T, 256, 0, s>>>((const bf16_t*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale, act);
+  const int ab = f32 ? 16 : 8;
+  if (act && rd == 0 && H * D % 4 == 0 && ldp % 4 == 0 && k_off % 4 == 0 && aligned_to(proj, ab) && aligned_to(qk, 16)) {
+    if (f32) lightning_prep_vec_kernel<float><<<T, 256, 0, s>>>((const float*)proj, ldp, k_off, qk, H * D, k_scale);
+    else lightning_prep_vec_kernel<bf16_t><<<T, 256, 0, s>>>((const bf16_t*)proj, ldp, k_off, qk, H * D, k_scale);
+    LWC_CHECK_LAUNCH();
+    return 0;
+  }
+#define LWC_PREP(AT, ACT) \
+  retention_prep_kernel<AT, ACT><<<T, 256, 0, s>>>((const AT*)proj, ldp, k_off, freq, mult, positions, qk, H, D, rd, k_scale)
+  if (f32 && act) LWC_PREP(float, true);
+  else if (f32) LWC_PREP(float, false);
+  else if (act) LWC_PREP(bf16_t, true);
+  else LWC_PREP(bf16_t, false);
+#undef LWC_PREP
   LWC_CHECK_LAUNCH();
   return 0;
 }
