@@ -15,16 +15,16 @@ int r32_xielu(const void*, int, const void*, void*, int, int, int, int, hipStrea
 int r32_residual_add_scaled(float*, const void*, float, long long, int, hipStream_t);
 int r32_residual_add_partials(float*, const float*, int, float, long long, hipStream_t);
 int r32_window_attn(const float*, const void*, const void*, long long, long long, int, const int*, const int*, int,
-                    const int*, int, const float*, const float*, const float*, int, int, void*, int, int, int, int, int, int, int,
+                    const int*, int, const float*, const float*, const float*, int, int, float, void*, int, int, int, int, int, int, int,
                     hipStream_t);
 int r32_window_attn_mfma_ok(int, int);
 int r32_window_attn_mfma(const float*, const void*, const void*, long long, long long, int, const int*, const int*,
-                         const int*, int, int, const int*, int, const float*, const float*, int, int, void*, int, int, int, int, int,
+                         const int*, int, int, const int*, int, const float*, const float*, int, int, float, void*, int, int, int, int, int,
                          hipStream_t);
 int r32_window_attn_decode_ok(int, int, int);
 int r32_window_attn_decode_splits(int, int, int, int, int);
 int r32_window_attn_decode(const float*, const void*, const void*, long long, long long, int, const int*, const int*, int,
-                           const float*, const float*, int, int, float*, float*, int, int, void*, int, int, int, int, int, int, int,
+                           const float*, const float*, int, int, float, float*, float*, int, int, void*, int, int, int, int, int, int, int,
                            hipStream_t);
 int r32_conv_hist(const void*, int, const float*, int, int, float*, long long, const int*, const int*, const int*,
                   const int*, void*, int, void*, int, int, int, int, int, int, int, hipStream_t);
@@ -56,7 +56,7 @@ int r32_post_norm(float*, const void*, int, float, const float*, void*, int, int
 int r32_post_norm_experts_ok(int);
 int r32_post_norm_experts(float*, const void*, const int*, const float*, int, const void*, int, const float*, int, float,
                           const float*, void*, int, int, float, int, hipStream_t);
-int r32_head_gate_rows(const void*, long long, long long, const void*, int, void*, int, int, int, int, int, hipStream_t);
+int r32_head_gate_rows(const void*, long long, long long, const void*, int, void*, int, int, int, int, int, int, hipStream_t);
 int r32_latent_kv_write(const void*, int, int, int, int, const float*, const float*, const float*, float, const int*,
                         const int*, void*, int, void*, void*, long long, long long, int, int, int, float, int, int,
                         hipStream_t);
@@ -68,7 +68,15 @@ int r32_retention_prep(const void*, int, int, const float*, float, const int*, f
 int r32_retention(const float*, const void*, int, const float*, float*, long long, const int*, const int*, const int*, float*,
                   int, int, int, int, int, int, int, hipStream_t);
 int r32_glu(const void*, int, void*, int, int, int, int, float, float, int, hipStream_t);
-int r32_gelu(const void*, int, void*, int, int, int, int, hipStream_t);
+int r32_act(const void*, int, void*, int, int, int, int, int, hipStream_t);
+int r32_hyper_max_streams();
+int r32_embed_streams(const void*, const int*, int, float, float, const float*, const float*, const float*, int, float, const float*,
+                      const float*, float*, void*, int, int, int, hipStream_t);
+int r32_hyper_step(float*, long long, int, const void*, int, const float*, const float*, float, const float*, const float*, void*,
+                   const long long*, int, int, int, int, hipStream_t);
+int r32_norm_rot_kv_write(const void*, int, const float*, const float*, const float*, const float*, float, int, const int*,
+                          const int*, float*, void*, void*, long long, long long, int, int, int, int, int, int, int, int, float,
+                          float, int, hipStream_t);
 int r32_rot_kv_write(const void*, int, const float*, const float*, const float*, float, int, const float*, const int*,
                      const int*, float*, void*, void*, long long, long long, int, int, int, int, int, int, float, float, int,
                      hipStream_t);
@@ -220,7 +228,7 @@ void residual_add_partials(Tensor x, Tensor parts, double m) {
 // sink: fp32 [H], exp(sink_h) joins head h's softmax denominator (no key, no value), or absent.
 void window_attn(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions, c10::optional<Tensor> cu_q,
                  Tensor block_tables, Tensor r1, Tensor r2, int64_t window, Tensor out, int64_t H, int64_t G,
-                 c10::optional<Tensor> sink, int64_t chunk) {
+                 c10::optional<Tensor> sink, int64_t chunk, double cap) {
   want(q, torch::kFloat32, "window_attn q");
   const int f = act_f32(k_cache, "window_attn k_cache");
   want(positions, torch::kInt32, "window_attn positions");
@@ -254,7 +262,7 @@ void window_attn(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions, c10
   }
   done(r32_window_attn(q.data_ptr<float>(), k_cache.data_ptr(), v_cache.data_ptr(), (long long)k_cache.stride(0),
                        (long long)v_cache.stride(0), BS, positions.data_ptr<int>(), cu, items, block_tables.data_ptr<int>(),
-                       width, r1.data_ptr<float>(), r2.data_ptr<float>(), sk, (int)window, (int)chunk, out.data_ptr(), ldo, T, (int)H, (int)G,
+                       width, r1.data_ptr<float>(), r2.data_ptr<float>(), sk, (int)window, (int)chunk, (float)cap, out.data_ptr(), ldo, T, (int)H, (int)G,
                        D, Dv, f, stream()), "window_attn");
 }
 
@@ -275,7 +283,7 @@ const float* sink_ptr(const c10::optional<Tensor>& sink, int64_t H, const char* 
 // Positions ascend by one along each item's rows.
 void window_attn_mfma(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions, Tensor cu_q, Tensor k_lens,
                       int64_t max_q, Tensor block_tables, c10::optional<Tensor> bias, int64_t window, Tensor out, int64_t H,
-                      int64_t G, c10::optional<Tensor> sink, int64_t chunk) {
+                      int64_t G, c10::optional<Tensor> sink, int64_t chunk, double cap) {
   want(q, torch::kFloat32, "window_attn_mfma q");
   want(positions, torch::kInt32, "window_attn_mfma positions");
   want(block_tables, torch::kInt32, "window_attn_mfma block_tables");
@@ -302,7 +310,7 @@ void window_attn_mfma(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions
                             (long long)v_cache.stride(0), BS, positions.data_ptr<int>(), cu_q.data_ptr<int>(),
                             k_lens.data_ptr<int>(), items, (int)max_q, block_tables.data_ptr<int>(),
                             (int)block_tables.size(1), bias.has_value() ? bias->data_ptr<float>() : nullptr,
-                            sink_ptr(sink, H, "window_attn_mfma"), (int)window, (int)chunk, out.data_ptr(), ldo, (int)H, (int)G, D, Dv,
+                            sink_ptr(sink, H, "window_attn_mfma"), (int)window, (int)chunk, (float)cap, out.data_ptr(), ldo, (int)H, (int)G, D, Dv,
                             stream()), "window_attn_mfma");
 }
 
@@ -310,7 +318,7 @@ void window_attn_mfma(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions
 // positions[b].  max_keys: a host-side upper bound of the keys a row sees (min(window, longest context)).
 void window_attn_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions, Tensor block_tables,
                         c10::optional<Tensor> bias, int64_t window, int64_t max_keys, Tensor out, int64_t H, int64_t G,
-                        c10::optional<Tensor> sink, bool values_in_keys, int64_t chunk) {
+                        c10::optional<Tensor> sink, bool values_in_keys, int64_t chunk, double cap) {
   want(q, torch::kFloat32, "window_attn_decode q");
   want(positions, torch::kInt32, "window_attn_decode positions");
   want(block_tables, torch::kInt32, "window_attn_decode block_tables");
@@ -336,7 +344,7 @@ void window_attn_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positio
   done(r32_window_attn_decode(q.data_ptr<float>(), k_cache.data_ptr(), v_cache.data_ptr(), (long long)k_cache.stride(0),
                               (long long)v_cache.stride(0), BS, positions.data_ptr<int>(), block_tables.data_ptr<int>(),
                               (int)block_tables.size(1), bias.has_value() ? bias->data_ptr<float>() : nullptr,
-                              sink_ptr(sink, H, "window_attn_decode"), (int)window, (int)chunk, po, po + (int64_t)B * H * S * Dv, S,
+                              sink_ptr(sink, H, "window_attn_decode"), (int)window, (int)chunk, (float)cap, po, po + (int64_t)B * H * S * Dv, S,
                               (int)max_keys, out.data_ptr(), ldo, B, (int)H, (int)G, D, Dv, values_in_keys ? 1 : 0, stream()),
        "window_attn_decode");
 }
@@ -729,16 +737,18 @@ void post_norm_experts(Tensor x, Tensor Y, Tensor inv, Tensor wts, c10::optional
                              (float)eps, fy | (fs << 1), stream()), "post_norm_experts");
 }
 
-// o [T, H, Dv] (unit last stride, any others), gate [T, H] logits (a column slice is fine), out [T, H Dv]
+// o [T, H, Dv] (unit last stride, any others), gate [T, H] or [T, H Dv] logits (a column slice is fine), out [T, H Dv]
 void head_gate_rows(Tensor o, Tensor gate, Tensor out) {
   const int f = act_f32(o, "head_gate_rows o");
   const int ldg = row_stride(gate, "head_gate_rows gate"), ldo = row_stride(out, "head_gate_rows out");
   TORCH_CHECK(o.is_cuda() && o.dim() == 3 && (o.stride(2) == 1 || o.size(2) == 1) && gate.scalar_type() == o.scalar_type() &&
                   out.scalar_type() == o.scalar_type() && gate.is_cuda() && out.is_cuda(), "head_gate_rows: dtypes");
   const int T = (int)o.size(0), H = (int)o.size(1), Dv = (int)o.size(2);
-  TORCH_CHECK(gate.size(0) == T && gate.size(1) == H && out.size(0) == T && out.size(1) == (int64_t)H * Dv, "head_gate_rows: shapes");
+  const bool entry = gate.size(1) != H;  // (one entry per head: both readings agree)
+  TORCH_CHECK(gate.size(0) == T && (!entry || gate.size(1) == (int64_t)H * Dv) && out.size(0) == T && out.size(1) == (int64_t)H * Dv,
+              "head_gate_rows: shapes");
   done(r32_head_gate_rows(o.data_ptr(), (long long)o.stride(0), (long long)o.stride(1), gate.data_ptr(), ldg, out.data_ptr(), ldo, T,
-                          H, Dv, f, stream()), "head_gate_rows");
+                          H, Dv, entry ? 1 : 0, f, stream()), "head_gate_rows");
 }
 
 // Low-rank attention, cache side: proj rows [dq (Cq) | c (C) | rotated key part (R) | ...]; cq [T, Cq] receives the
@@ -868,13 +878,13 @@ void glu(Tensor in, Tensor out, int64_t mode, double alpha, double limit) {
                f, stream()), "glu");
 }
 
-// out = z / 2 (1 + erf(z / sqrt 2)) over row-dense views of one dtype
-void gelu(Tensor in, Tensor out) {
-  const int f = act_f32(in, "gelu in");
-  const int ldi = row_stride(in, "gelu in"), ldo = row_stride(out, "gelu out");
-  TORCH_CHECK(out.is_cuda() && out.scalar_type() == in.scalar_type() && out.size(0) == in.size(0) && out.size(1) == in.size(1),
-              "gelu: shapes or dtypes disagree");
-  done(r32_gelu(in.data_ptr(), ldi, out.data_ptr(), ldo, (int)in.size(0), (int)in.size(1), f, stream()), "gelu");
+// out = f(z) over row-dense views of one dtype; kind 0: z / 2 (1 + erf(z / sqrt 2)), 1: max(z, 0)^2
+void act(Tensor in, Tensor out, int64_t kind) {
+  const int f = act_f32(in, "act in");
+  const int ldi = row_stride(in, "act in"), ldo = row_stride(out, "act out");
+  TORCH_CHECK(out.is_cuda() && out.scalar_type() == in.scalar_type() && out.size(0) == in.size(0) && out.size(1) == in.size(1) &&
+                  (kind == 0 || kind == 1), "act: shapes or dtypes disagree");
+  done(r32_act(in.data_ptr(), ldi, out.data_ptr(), ldo, (int)in.size(0), (int)in.size(1), (int)kind, f, stream()), "act");
 }
 
 const float* opt_f32(const c10::optional<Tensor>& t, int64_t n, const char* name) {
@@ -910,6 +920,86 @@ void rot_kv_write(Tensor src, c10::optional<Tensor> wq, c10::optional<Tensor> wk
                         positions.data_ptr<int>(), slots.data_ptr<int>(), q_out.data_ptr<float>(), k_cache.data_ptr(),
                         v_cache.data_ptr(), (long long)k_cache.stride(0), (long long)v_cache.stride(0), BS, T, (int)H, (int)G, D,
                         Dv, (float)eps, (float)scale, fi | (fc << 1), stream()), "rot_kv_write");
+}
+
+// src rows [q (H D) | k (G D) | v (G Dv)] (bf16 or fp32); bias fp32 per column or absent; wq fp32 [H D] / wk fp32 [G D]:
+// weights of the RMS norm over the whole projection, or absent; q_out fp32 [T, H, Dk >= D]; caches (absent with G = 0: only q,
+// a layer that reads another layer's keys and values): one layer's views, head sizes Dk and >= Dv, padded with zeros.
+void norm_rot_kv_write(Tensor src, c10::optional<Tensor> bias, c10::optional<Tensor> wq, c10::optional<Tensor> wk,
+                       c10::optional<Tensor> freq, double mult, int64_t rd, Tensor positions, Tensor slots, Tensor q_out,
+                       c10::optional<Tensor> k_cache, c10::optional<Tensor> v_cache, int64_t H, int64_t G, int64_t D, int64_t Dv,
+                       double eps, double scale) {
+  const int fi = act_f32(src, "norm_rot_kv_write src");
+  const int lds = row_stride(src, "norm_rot_kv_write src"), T = (int)src.size(0);
+  want(positions, torch::kInt32, "norm_rot_kv_write positions");
+  want(slots, torch::kInt32, "norm_rot_kv_write slots");
+  want(q_out, torch::kFloat32, "norm_rot_kv_write q_out");
+  TORCH_CHECK(H > 0 && G >= 0 && D > 0 && Dv >= 0 && q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == H && q_out.size(2) >= D &&
+                  src.size(1) == H * D + G * (D + Dv) && positions.numel() == T && slots.numel() == T && rd >= 0 && rd <= D &&
+                  rd % 2 == 0 && (rd == 0 || freq.has_value()), "norm_rot_kv_write: shapes disagree");
+  const int Dk = (int)q_out.size(2);
+  int NB, BS = 1, nk, nv, fc = fi, Dvp = (int)Dv;
+  void *kp = nullptr, *vp = nullptr;
+  long long kb = 0, vb = 0;
+  if (G > 0) {
+    TORCH_CHECK(k_cache.has_value() && v_cache.has_value(), "norm_rot_kv_write: caches missing");
+    fc = act_f32(*k_cache, "norm_rot_kv_write k_cache");
+    TORCH_CHECK(v_cache->is_cuda() && v_cache->scalar_type() == k_cache->scalar_type() && (fi || !fc),
+                "norm_rot_kv_write: caches of one dtype, bf16 rows only into a bf16 cache");
+    cache_layout(*k_cache, *v_cache, NB, BS, nk, nv, "norm_rot_kv_write");
+    TORCH_CHECK(H % G == 0 && nk == G * Dk && nv % G == 0 && nv / G >= Dv, "norm_rot_kv_write: cache sizes");
+    Dvp = nv / (int)G;
+    kp = k_cache->data_ptr(), vp = v_cache->data_ptr();
+    kb = (long long)k_cache->stride(0), vb = (long long)v_cache->stride(0);
+  }
+  done(r32_norm_rot_kv_write(src.data_ptr(), lds, opt_f32(bias, src.size(1), "norm_rot_kv_write bias"),
+                             opt_f32(wq, H * D, "norm_rot_kv_write wq"), opt_f32(wk, G * D, "norm_rot_kv_write wk"),
+                             opt_f32(freq, rd / 2, "norm_rot_kv_write freq"), (float)mult, (int)rd, positions.data_ptr<int>(),
+                             slots.data_ptr<int>(), q_out.data_ptr<float>(), kp, vp, kb, vb, BS, T, (int)H, (int)G, (int)D, (int)Dv,
+                             Dk, Dvp, (float)eps, (float)scale, fi | (fc << 1), stream()), "norm_rot_kv_write");
+}
+
+int64_t hyper_max_streams() { return r32_hyper_max_streams(); }
+
+// X fp32 [S, T, d] <- dyt_e(table[tokens] * scale) in every stream; h [T, d] (the table's dtype) <- dyt(sum_s in_s X_s)
+void embed_streams(Tensor table, Tensor tokens, double scale, double ae, Tensor we, Tensor be, Tensor in, double a, Tensor w, Tensor b,
+                   Tensor X, Tensor h) {
+  const int f = act_f32(table, "embed_streams table");
+  want(tokens, torch::kInt32, "embed_streams tokens");
+  want(X, torch::kFloat32, "embed_streams X");
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && X.dim() == 3, "embed_streams: table [V, d], X [S, T, d]");
+  const int T = (int)tokens.numel(), d = (int)table.size(1), S = (int)X.size(0);
+  TORCH_CHECK(X.size(1) == T && X.size(2) == d && S <= r32_hyper_max_streams() && h.is_cuda() && h.is_contiguous() &&
+                  h.scalar_type() == table.scalar_type() && h.numel() == (int64_t)T * d, "embed_streams: shapes disagree");
+  done(r32_embed_streams(table.data_ptr(), tokens.data_ptr<int>(), (int)table.size(0), (float)scale, (float)ae,
+                         opt_f32(we, d, "embed_streams we"), opt_f32(be, d, "embed_streams be"), opt_f32(in, S, "embed_streams in"), S,
+                         (float)a, opt_f32(w, d, "embed_streams w"), opt_f32(b, d, "embed_streams b"), X.data_ptr<float>(),
+                         h.data_ptr(), T, d, f | (f << 1), stream()), "embed_streams");
+}
+
+// X fp32 [S, T, d]: X'_t = sum_s mix[s][t] X_s + out[t] (y + bias) (stored when write), h = dyt(sum_t in[t] X'_t); coef fp32
+// [S S + 2 S] = mix | out | in; y [T, d]; rows (int64, not with write): only these rows, h [len(rows), d]
+void hyper_step(Tensor X, Tensor y, c10::optional<Tensor> bias, Tensor coef, double a, Tensor w, Tensor b, Tensor h,
+                c10::optional<Tensor> rows, bool write) {
+  want(X, torch::kFloat32, "hyper_step X");
+  want(coef, torch::kFloat32, "hyper_step coef");
+  const int fy = act_f32(y, "hyper_step y"), fh = act_f32(h, "hyper_step h");
+  const int ldy = row_stride(y, "hyper_step y");
+  TORCH_CHECK(X.dim() == 3 && h.dim() == 2 && h.is_contiguous(), "hyper_step: X [S, T, d], h [n, d]");
+  const int S = (int)X.size(0), T = (int)X.size(1), d = (int)X.size(2);
+  const long long* rp = nullptr;
+  int n = T;
+  if (rows.has_value()) {
+    want(*rows, torch::kInt64, "hyper_step rows");
+    TORCH_CHECK(!write, "hyper_step: a row list leaves the streams as they are");
+    n = (int)rows->numel();
+    rp = (const long long*)rows->data_ptr<int64_t>();
+  }
+  TORCH_CHECK(S >= 1 && S <= r32_hyper_max_streams() && coef.numel() == (int64_t)S * S + 2 * S && y.size(0) == T && y.size(1) == d &&
+                  h.size(0) == n && h.size(1) == d, "hyper_step: shapes disagree");
+  done(r32_hyper_step(X.data_ptr<float>(), (long long)T * d, S, y.data_ptr(), ldy, opt_f32(bias, d, "hyper_step bias"),
+                      coef.data_ptr<float>(), (float)a, opt_f32(w, d, "hyper_step w"), opt_f32(b, d, "hyper_step b"), h.data_ptr(), rp,
+                      n, d, write ? 1 : 0, fy | (fh << 1), stream()), "hyper_step");
 }
 
 // o, out [T, H Dv] row-dense views of one dtype (not the same memory); g [T, >= H] gate logits or absent
@@ -1036,8 +1126,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("retention", &retention);
   m.def("retention_max_dim", &retention_max_dim);
   m.def("glu", &glu);
-  m.def("gelu", &gelu);
+  m.def("act", &act);
   m.def("rot_kv_write", &rot_kv_write);
+  m.def("norm_rot_kv_write", &norm_rot_kv_write);
+  m.def("hyper_max_streams", &hyper_max_streams);
+  m.def("embed_streams", &embed_streams);
+  m.def("hyper_step", &hyper_step);
   m.def("head_gate_unrotate", &head_gate_unrotate);
   m.def("add_rmsnorm", &add_rmsnorm);
   m.def("chan_rule", &chan_rule);

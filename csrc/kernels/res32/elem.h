@@ -36,6 +36,10 @@ inline bool aligned_to(const void* p, int bytes) { return ((uintptr_t)p & (uintp
 LWC_DEVICE float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 LWC_DEVICE float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
 LWC_DEVICE float silu_f(float x) { return x / (1.0f + expf(-x)); }
+// c tanh(x / c) as c - 2 c / (exp2(k x) + 1), k = 2 log2(e) / c (absolute error ~1e-7 c; exp2 overflowing to infinity gives c)
+LWC_DEVICE float softcap_f(float x, float c, float k) {
+  return c - 2.0f * c * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(k * x) + 1.0f);
+}
 LWC_DEVICE float gelu_tanh_f(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }

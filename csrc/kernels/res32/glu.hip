@@ -4,7 +4,8 @@
 //   mode 1   g' = min(g, L), u' = clamp(u, -L, L);  y = g' * sigmoid(alpha g') * (u' + 1)      (clamped gate unit)
 // in: rows [gate (n) | up (n)] with leading dimension ldi; out: rows of n (leading dimension ldo).
 //
-//   gelu     y = z / 2 (1 + erf(z / sqrt(2))) over rows of n (an ungated feed-forward's activation)
+//   act      over rows of n, an ungated feed-forward's activation:  kind 0 (gelu) y = z / 2 (1 + erf(z / sqrt(2)));
+//            kind 1 (relu2) y = max(z, 0)^2
 #include "elem.h"
 
 namespace lwc {
@@ -58,23 +59,30 @@ template <> struct Gelu<bf16_t> {
   }
 };
 
-template <typename AT>
-__global__ void gelu_kernel(const AT* __restrict__ in, int ldi, AT* __restrict__ out, int ldo, int n, long long total) {
+template <typename AT> struct Relu2 {
+  static LWC_DEVICE float f(float z) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  }
+};
+
+template <typename AT, typename F>
+__global__ void act_kernel(const AT* __restrict__ in, int ldi, AT* __restrict__ out, int ldo, int n, long long total) {
   for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < total; e += (long long)gridDim.x * blockDim.x) {
     const long long t = e / n;
     const int c = (int)(e - t * n);
-    Elem<AT>::st(out + t * ldo + c, Gelu<AT>::f(Elem<AT>::ld(in + t * ldi + c)));
+    Elem<AT>::st(out + t * ldo + c, F::f(Elem<AT>::ld(in + t * ldi + c)));
   }
 }
 
 // four columns per thread, rows along the grid's second dimension (no division per element)
-template <typename AT>
-__global__ void gelu_vec_kernel(const AT* __restrict__ in, int ldi, AT* __restrict__ out, int ldo, int n4, int T) {
+template <typename AT, typename F>
+__global__ void act_vec_kernel(const AT* __restrict__ in, int ldi, AT* __restrict__ out, int ldo, int n4, int T) {
   const int c = 4 * (blockIdx.x * blockDim.x + threadIdx.x);
   if (c >= 4 * n4) return;
   for (int t = blockIdx.y; t < T; t += gridDim.y) {
     const float4v z = Vec4<AT>::ld(in + (size_t)t * ldi + c);
-    Vec4<AT>::st(out + (size_t)t * ldo + c, float4v{Gelu<AT>::f(z[0]), Gelu<AT>::f(z[1]), Gelu<AT>::f(z[2]), Gelu<AT>::f(z[3])});
+    Vec4<AT>::st(out + (size_t)t * ldo + c, float4v{F::f(z[0]), F::f(z[1]), F::f(z[2]), F::f(z[3])});
   }
 }
 
@@ -119,16 +127,28 @@ extern "C" int r32_glu(const void* in, int ldi, void* out, int ldo, int T, int n
   return 0;
 }
 
-extern "C" int r32_gelu(const void* in, int ldi, void* out, int ldo, int T, int n, int f32, hipStream_t s) {
+// kind: 0 gelu (erf form), 1 relu squared
+extern "C" int r32_act(const void* in, int ldi, void* out, int ldo, int T, int n, int kind, int f32, hipStream_t s) {
   const long long total = (long long)T * n;
   if (total <= 0) return 0;
   const int ab = f32 ? 16 : 8;
   const bool vec = n % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && aligned_to(in, ab) && aligned_to(out, ab);
   const dim3 vgrid((n / 4 + 255) / 256, T < 32768 ? T : 32768);
-  if (vec && f32) gelu_vec_kernel<float><<<vgrid, 256, 0, s>>>((const float*)in, ldi, (float*)out, ldo, n / 4, T);
-  else if (vec) gelu_vec_kernel<bf16_t><<<vgrid, 256, 0, s>>>((const bf16_t*)in, ldi, (bf16_t*)out, ldo, n / 4, T);
-  else if (f32) gelu_kernel<float><<<glu_grid(total), 256, 0, s>>>((const float*)in, ldi, (float*)out, ldo, n, total);
-  else gelu_kernel<bf16_t><<<glu_grid(total), 256, 0, s>>>((const bf16_t*)in, ldi, (bf16_t*)out, ldo, n, total);
+#define LWC_ACT(AT, F)                                                                                              \
+  if (vec) act_vec_kernel<AT, F<AT>><<<vgrid, 256, 0, s>>>((const AT*)in, ldi, (AT*)out, ldo, n / 4, T);            \
+  else act_kernel<AT, F<AT>><<<glu_grid(total), 256, 0, s>>>((const AT*)in, ldi, (AT*)out, ldo, n, total)
+  if (kind == 0 && f32) {
+    LWC_ACT(float, Gelu);
+  } else if (kind == 0) {
+    LWC_ACT(bf16_t, Gelu);
+  } else if (kind == 1 && f32) {
+    LWC_ACT(float, Relu2);
+  } else if (kind == 1) {
+    LWC_ACT(bf16_t, Relu2);
+  } else {
+    return -1;
+  }
+#undef LWC_ACT
   LWC_CHECK_LAUNCH();
   return 0;
 }

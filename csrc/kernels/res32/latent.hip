@@ -12,8 +12,9 @@
 //   latent_q_rows     the fp32 query rows [ qn * scale (C) | rot(q_rot) * scale (R) | 0 ] per head from the absorbed
 //                     unrotated part qn ([H, T, C] fp32) and the up-projected query rows (rotated part of every head)
 //
-//   head_gate_rows    out[t, h, :] = o[t, h, :] * sigmoid(gate[t, h]): one gate per head on the attention's result, from
-//                     whatever strides the up-projection left it in ([H, T, Dv] of a batched product, padded heads)
+//   head_gate_rows    out[t, h, :] = o[t, h, :] * sigmoid(gate[t, h]) (one gate per head) or * sigmoid(gate[t, h, :]) (one per
+//                     entry), from whatever strides the attention's result lies in ([H, T, Dv] of a batched product, padded
+//                     heads)
 //
 // Rotation ("interleaved"): entries (2i, 2i + 1) at position p turn by the angle a = p * f_i (fp32 product of the
 // position and the fp32 frequency), (u, v) -> m (u cos a - v sin a, v cos a + u sin a); f and m come from the host
@@ -129,28 +130,35 @@ latent_expand_write_kernel(const AT* __restrict__ kv, int ldk, const AT* __restr
   }
 }
 
-template <typename AT>
+// ENTRY: a gate per entry (gate rows [H Dv]), else per head (gate rows [H])
+template <typename AT, bool ENTRY>
 __global__ void __launch_bounds__(256) head_gate_rows_kernel(const AT* __restrict__ o, long long row_stride, long long head_stride,
                                                               const AT* __restrict__ gate, int ldg, AT* __restrict__ out, int ldo,
                                                               int H, int Dv) {
   const int t = blockIdx.x;
   for (int e = threadIdx.x; e < H * Dv; e += blockDim.x) {
     const int h = e / Dv, i = e - h * Dv;
-    const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + h));
+    const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + (ENTRY ? e : h)));
     Elem<AT>::st(out + (size_t)t * ldo + e, Elem<AT>::ld(o + t * row_stride + h * head_stride + i) * g);
   }
 }
 
 // four entries per thread: Dv, every stride and every base a multiple of four entries
-template <typename AT>
+template <typename AT, bool ENTRY>
 __global__ void __launch_bounds__(256) head_gate_rows_vec_kernel(const AT* __restrict__ o, long long row_stride,
                                                                   long long head_stride, const AT* __restrict__ gate, int ldg,
                                                                   AT* __restrict__ out, int ldo, int H, int dv4) {
   const int t = blockIdx.x;
   for (int e = threadIdx.x; e < H * dv4; e += blockDim.x) {
     const int h = e / dv4, i = 4 * (e - h * dv4);
-    const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + h));
-    Vec4<AT>::st(out + (size_t)t * ldo + 4 * e, Vec4<AT>::ld(o + t * row_stride + h * head_stride + i) * g);
+    const float4v x = Vec4<AT>::ld(o + t * row_stride + h * head_stride + i);
+    if constexpr (ENTRY) {
+      const float4v z = Vec4<AT>::ld(gate + (size_t)t * ldg + 4 * e);
+      Vec4<AT>::st(out + (size_t)t * ldo + 4 * e, x * float4v{sigmoid_f(z[0]), sigmoid_f(z[1]), sigmoid_f(z[2]), sigmoid_f(z[3])});
+    } else {
+      const float g = sigmoid_f(Elem<AT>::ld(gate + (size_t)t * ldg + h));
+      Vec4<AT>::st(out + (size_t)t * ldo + 4 * e, x * g);
+    }
   }
 }
 
@@ -159,21 +167,27 @@ __global__ void __launch_bounds__(256) head_gate_rows_vec_kernel(const AT* __res
 
 using namespace lwc;
 
+// entry: gate rows of H * Dv logits, else of H
 extern "C" int r32_head_gate_rows(const void* o, long long row_stride, long long head_stride, const void* gate, int ldg, void* out,
-                                  int ldo, int T, int H, int Dv, int f32, hipStream_t s) {
+                                  int ldo, int T, int H, int Dv, int entry, int f32, hipStream_t s) {
   if (T <= 0) return 0;
   const int ab = f32 ? 16 : 8;
-  const bool vec = Dv % 4 == 0 && row_stride % 4 == 0 && head_stride % 4 == 0 && ldo % 4 == 0 && aligned_to(o, ab) && aligned_to(out, ab);
-#define LWC_HGR(AT)                                                                                                        \
-  if (vec)                                                                                                                 \
-    head_gate_rows_vec_kernel<AT><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, \
-                                                    ldo, H, Dv / 4);                                                       \
-  else                                                                                                                     \
-    head_gate_rows_kernel<AT><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, ldo, H, Dv)
-  if (f32) {
-    LWC_HGR(float);
+  const bool vec = Dv % 4 == 0 && row_stride % 4 == 0 && head_stride % 4 == 0 && ldo % 4 == 0 && aligned_to(o, ab) && aligned_to(out, ab) &&
+                   (!entry || (ldg % 4 == 0 && aligned_to(gate, ab)));
+#define LWC_HGR(AT, E)                                                                                                        \
+  if (vec)                                                                                                                    \
+    head_gate_rows_vec_kernel<AT, E><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, \
+                                                       ldo, H, Dv / 4);                                                       \
+  else                                                                                                                        \
+    head_gate_rows_kernel<AT, E><<<T, 256, 0, s>>>((const AT*)o, row_stride, head_stride, (const AT*)gate, ldg, (AT*)out, ldo, H, Dv)
+  if (f32 && entry) {
+    LWC_HGR(float, true);
+  } else if (f32) {
+    LWC_HGR(float, false);
+  } else if (entry) {
+    LWC_HGR(bf16_t, true);
   } else {
-    LWC_HGR(bf16_t);
+    LWC_HGR(bf16_t, false);
   }
 #undef LWC_HGR
   LWC_CHECK_LAUNCH();

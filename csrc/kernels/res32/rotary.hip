@@ -6,6 +6,10 @@
 //                       (u c - v s, v c + u s), c = mult cos(p f_i), s = mult sin(p f_i);
 //                       q times `scale` -> fp32 [T, H*D]; k -> paged K cache; v, optionally rotated the same way over
 //                       all Dv entries by its own frequencies (no multiplier) -> 4-token interleaved paged V cache
+//   norm_rot_kv_write   the same for layers whose q and k are RMS-normed over their WHOLE projections (a weight per row of
+//                       the projection): rows [q | k | v] plus an optional bias per column; heads may be padded with zeros
+//                       in q_out and in the cache (sizes the attention kernels are built for); without k and v (G = 0) for a
+//                       layer that reads another layer's cache
 //   head_gate_unrotate  out[t, h, :] = rot(o[t, h, :], -p) * sigmoid(g[t, h]) * scale: an attention output over rotated
 //                       values turned back by the query's position, one gate per head (rotation optional)
 //   add_rmsnorm         x (fp32) += y;  out = x / rms(x) * w: the residual sum and the next sublayer's input norm
@@ -188,6 +192,133 @@ __global__ void __launch_bounds__(256) rot_kv_write_vec_kernel(
   }
 }
 
+struct NormRotParams {
+  const void* src;
+  int lds;
+  const float *bias, *wq, *wk, *freq;  // bias [nq + nk + nv], wq [H D] and wk [G D] may be null
+  float mult;
+  int rd;
+  const int *positions, *slots;
+  float* q_out;                        // [T, H, Dk]
+  void *k_cache, *v_cache;             // head sizes Dk and Dvp
+  long long kb_stride, vb_stride;
+  int block_size, H, G, D, Dv, Dk, Dvp;
+  float eps, scale;
+};
+
+// One entry of a padded head (H heads of q, then G of k): normed with the projection's factor, rotated, 0 beyond D
+template <typename IT, typename CT>
+__global__ void __launch_bounds__(256) norm_rot_kv_write_kernel(const NormRotParams p) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, H = p.H, G = p.G, D = p.D, Dv = p.Dv, Dk = p.Dk, Dvp = p.Dvp, half = p.rd >> 1;
+  const IT* pr = (const IT*)p.src + (size_t)t * p.lds;
+  const float pos = (float)p.positions[t];
+  const int slot = G > 0 ? p.slots[t] : -1;
+  const bool write = slot >= 0;
+  const long long blk = write ? slot / p.block_size : 0, off = write ? slot % p.block_size : 0;
+  const int nq = H * D, nk = G * D, nv = G * Dvp;
+  auto ld = [&](int i) { return Elem<IT>::ld(pr + i) + (p.bias ? p.bias[i] : 0.f); };
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x; i < nq; i += blockDim.x) {
+    const float v = ld(i);
+    sq += v * v;
+  }
+  for (int i = threadIdx.x; i < nk; i += blockDim.x) {
+    const float v = ld(nq + i);
+    sk += v * v;
+  }
+  const float rq = p.wq ? 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + p.eps) : 1.0f;
+  const float rk = p.wk && nk ? 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + p.eps) : 1.0f;
+  for (int e = threadIdx.x; e < (H + (write ? G : 0)) * Dk; e += blockDim.x) {
+    const int h = e / Dk, i = e - h * Dk;
+    const bool isq = h < H;
+    const float* w = isq ? p.wq : p.wk;
+    const int base = h * D, wb = isq ? base : base - nq;  // (the k heads follow the q heads)
+    const float r = isq ? rq : rk;
+    float x = 0.f;
+    if (i < D) {
+      x = ld(base + i) * (w ? r * w[wb + i] : 1.0f);
+      if (i < p.rd) {
+        const bool first = i < half;
+        const int m = first ? i : i - half, j = first ? i + half : i - half;
+        const float xp = ld(base + j) * (w ? r * w[wb + j] : 1.0f);
+        float sn, cs;
+        sincosf(pos * p.freq[m], &sn, &cs);
+        sn *= p.mult, cs *= p.mult;
+        x = first ? x * cs - xp * sn : x * cs + xp * sn;
+      }
+    }
+    if (isq) p.q_out[((size_t)t * H + h) * Dk + i] = x * p.scale;
+    else Elem<CT>::st((CT*)p.k_cache + blk * p.kb_stride + off * ((long long)G * Dk) + (h - H) * Dk + i, x);
+  }
+  if (!write) return;
+  CT* vc = (CT*)p.v_cache + blk * p.vb_stride + (off >> 2) * (4LL * nv) + (off & 3);  // 4-token interleaved
+  for (int e = threadIdx.x; e < nv; e += blockDim.x) {
+    const int g = e / Dvp, i = e - g * Dvp;
+    Elem<CT>::st(vc + 4LL * e, i < Dv ? ld(nq + nk + g * Dv + i) : 0.f);
+  }
+}
+
+// D, Dv, Dk, Dvp multiples of four, rd a multiple of eight, every base a multiple of four entries
+template <typename IT, typename CT>
+__global__ void __launch_bounds__(256) norm_rot_kv_write_vec_kernel(const NormRotParams p) {
+  extern __shared__ __attribute__((aligned(16))) float tab[];  // [rd] angles
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, H = p.H, G = p.G, D = p.D, Dv = p.Dv, half = p.rd >> 1;
+  const IT* pr = (const IT*)p.src + (size_t)t * p.lds;
+  const int slot = G > 0 ? p.slots[t] : -1;
+  const bool write = slot >= 0;
+  const long long blk = write ? slot / p.block_size : 0, off = write ? slot % p.block_size : 0;
+  const int nq = H * D, nk = G * D, nv = G * p.Dvp;
+  auto ld = [&](int i) {
+    float4v x = Vec4<IT>::ld(pr + i);
+    if (p.bias) x += Vec4<float>::ld(p.bias + i);
+    return x;
+  };
+  auto sum2 = [](const float4v& v) { return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; };
+  if (p.rd) angle_table(tab, p.freq, half, p.mult, (float)p.positions[t]);
+  float sq = 0.f, sk = 0.f;
+  if (p.wq)
+    for (int i = threadIdx.x * 4; i < nq; i += blockDim.x * 4) sq += sum2(ld(i));
+  if (p.wk && write)
+    for (int i = threadIdx.x * 4; i < nk; i += blockDim.x * 4) sk += sum2(ld(nq + i));
+  // (block_sum's barriers also publish the angle table)
+  const float rq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + p.eps);
+  const float rk = p.wk && write ? 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + p.eps) : 1.0f;
+  const int k4 = p.Dk >> 2, v4 = p.Dvp >> 2, uk = (H + (write ? G : 0)) * k4, uv = write ? G * v4 : 0;
+  for (int u = threadIdx.x; u < uk + uv; u += blockDim.x) {
+    if (u < uk) {
+      const int h = u / k4, i = (u - h * k4) * 4;
+      const bool isq = h < H;
+      const float* w = isq ? p.wq : p.wk;
+      const int base = h * D, wb = isq ? base : base - nq;  // (the k heads follow the q heads)
+      const float r = isq ? rq : rk;
+      float4v x = float4v{0.f, 0.f, 0.f, 0.f};
+      if (i < D) {
+        x = ld(base + i);
+        if (w) x *= Vec4<float>::ld(w + wb + i) * r;
+        if (i < p.rd) {
+          const bool first = i < half;
+          const int m = first ? i : i - half, j = first ? i + half : i - half;
+          float4v xp = ld(base + j);
+          if (w) xp *= Vec4<float>::ld(w + wb + j) * r;
+          const float4v cs = Vec4<float>::ld(tab + m), sn = Vec4<float>::ld(tab + half + m);
+          x = first ? x * cs - xp * sn : x * cs + xp * sn;
+        }
+      }
+      if (isq) Vec4<float>::st(p.q_out + ((size_t)t * H + h) * p.Dk + i, x * p.scale);
+      else Vec4<CT>::st((CT*)p.k_cache + blk * p.kb_stride + off * ((long long)G * p.Dk) + (h - H) * p.Dk + i, x);
+    } else {
+      const int e = u - uk, g = e / v4, i = (e - g * v4) * 4;
+      const float4v x = i < Dv ? ld(nq + nk + g * Dv + i) : float4v{0.f, 0.f, 0.f, 0.f};
+      // V is 4-token interleaved: [block][offset / 4][column][offset % 4]
+      CT* vc = (CT*)p.v_cache + blk * p.vb_stride + (off >> 2) * (4LL * nv) + (off & 3) + 16LL * e;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) Elem<CT>::st(vc + 4 * c, x[c]);
+    }
+  }
+}
+
 template <typename AT>
 __global__ void __launch_bounds__(256) head_gate_unrotate_vec_kernel(const AT* __restrict__ o, int ldi, const AT* __restrict__ g,
                                                                       int ldg, const float* __restrict__ vfreq,
@@ -291,6 +422,40 @@ extern "C" int r32_rot_kv_write(const void* src, int lds, const float* wq, const
     return -1;
   }
 #undef LWC_ROT
+  LWC_CHECK_LAUNCH();
+  return 0;
+}
+
+// io: bit 0 = rows fp32 (else bf16), bit 1 = cache fp32 (else bf16).  G = 0: only q (k_cache, v_cache, slots unused); bias,
+// wq, wk may be null (no bias, no norm); freq may be null when rd == 0.
+extern "C" int r32_norm_rot_kv_write(const void* src, int lds, const float* bias, const float* wq, const float* wk,
+                                     const float* freq, float mult, int rd, const int* positions, const int* slots, float* q_out,
+                                     void* k_cache, void* v_cache, long long kb_stride, long long vb_stride, int block_size, int T,
+                                     int H, int G, int D, int Dv, int Dk, int Dvp, float eps, float scale, int io, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (H < 1 || G < 0 || rd < 0 || rd > D || (rd & 1) || (rd > 0 && !freq) || Dk < D || Dvp < Dv) return -1;
+  NormRotParams p;
+  p.src = src; p.lds = lds; p.bias = bias; p.wq = wq; p.wk = wk; p.freq = freq; p.mult = mult; p.rd = rd; p.positions = positions;
+  p.slots = slots; p.q_out = q_out; p.k_cache = k_cache; p.v_cache = v_cache; p.kb_stride = kb_stride; p.vb_stride = vb_stride;
+  p.block_size = block_size; p.H = H; p.G = G; p.D = D; p.Dv = Dv; p.Dk = Dk; p.Dvp = Dvp; p.eps = eps; p.scale = scale;
+  const int ib = (io & 1) ? 16 : 8, cb = (io & 2) ? 16 : 8;
+  const bool vec = D % 4 == 0 && Dv % 4 == 0 && Dk % 4 == 0 && Dvp % 4 == 0 && rd % 8 == 0 && lds % 4 == 0 && kb_stride % 4 == 0 &&
+                   aligned_to(src, ib) && aligned_to(k_cache, cb) && aligned_to(q_out, 16) && aligned_to(bias, 16) &&
+                   aligned_to(wq, 16) && aligned_to(wk, 16);
+  const size_t shm = (size_t)(rd ? rd : 4) * sizeof(float);
+#define LWC_NRK(IT, CT)                                          \
+  if (vec) norm_rot_kv_write_vec_kernel<IT, CT><<<T, 256, shm, s>>>(p); \
+  else norm_rot_kv_write_kernel<IT, CT><<<T, 256, 0, s>>>(p)
+  if (io == 3) {
+    LWC_NRK(float, float);
+  } else if (io == 0) {
+    LWC_NRK(bf16_t, bf16_t);
+  } else if (io == 1) {
+    LWC_NRK(float, bf16_t);
+  } else {
+    return -1;
+  }
+#undef LWC_NRK
   LWC_CHECK_LAUNCH();
   return 0;
 }

@@ -3,7 +3,7 @@
 //   score(i, j) = q_i . k_j - r1_h * ln(1 + r2_h * (i - j))        for 0 <= i - j < window
 //   out_i       = softmax_j(score) . v_j
 // With a sink (fp32 per head) the softmax's denominator also holds exp(sink_h): a share of the weight that belongs
-// to no key and adds no value.
+// to no key and adds no value.  With a cap c > 0 a score q . k becomes c tanh(q . k / c) (before the distance bias).
 // q arrives in fp32 already multiplied by the head's softmax scale; K rows have D elements, V rows Dv (any sizes,
 // D != Dv allowed), G key/value heads serve H query heads (head h reads group h / (H / G)).  Scores, the softmax
 // and the weighted sum are fp32 whatever the cache's element type (bf16 or fp32).
@@ -19,7 +19,7 @@
 //
 // window_attn_kernel: one wave per (row, head); lanes over 64 keys for the scores, an online softmax per
 // 64-key step, then lanes over the value dimension (several keys side by side when Dv < 64).
-#include "../common.h"
+#include "elem.h"
 
 namespace lwc {
 namespace {
@@ -71,7 +71,7 @@ window_attn_kernel(const float* __restrict__ q, const CT* __restrict__ k_cache, 
                    long long kb_stride, long long vb_stride, int block_size, const int* __restrict__ positions,
                    const int* __restrict__ cu_q, int n_items, const int* __restrict__ block_tables, int bt_width,
                    const float* __restrict__ r1, const float* __restrict__ r2, const float* __restrict__ sink, int window,
-                   int chunk, CT* __restrict__ out, int ldo, int H, int G, int D, int Dv) {
+                   int chunk, float cap, CT* __restrict__ out, int ldo, int H, int G, int D, int Dv) {
   extern __shared__ float q_s[];  // [D]
   __shared__ float p_s[64];
   __shared__ long long vo_s[64];
@@ -111,7 +111,9 @@ window_attn_kernel(const float* __restrict__ q, const CT* __restrict__ k_cache, 
       const long long blk = table[j / block_size];
       const long long off = j % block_size;
       const CT* kr = k_cache + blk * kb_stride + (off * G + g) * D;
-      s = KLoad<CT>::dot(kr, q_s, D) - r1h * log1pf(r2h * (float)(i - j));
+      s = KLoad<CT>::dot(kr, q_s, D);
+      if (cap > 0.f) s = cap * tanhf(s / cap);
+      s -= r1h * log1pf(r2h * (float)(i - j));
       vo = blk * vb_stride + (off >> 2) * (4LL * G * Dv) + 4LL * g * Dv + (off & 3);
     }
     const float m_new = fmaxf(m, wave_max(s));
@@ -162,7 +164,8 @@ using namespace lwc;
 extern "C" int r32_window_attn(const float* q, const void* k_cache, const void* v_cache, long long kb_stride,
                                long long vb_stride, int block_size, const int* positions, const int* cu_q, int n_items,
                                const int* block_tables, int bt_width, const float* r1, const float* r2, const float* sink,
-                               int window, int chunk, void* out, int ldo, int T, int H, int G, int D, int Dv, int f32, hipStream_t s) {
+                               int window, int chunk, float cap, void* out, int ldo, int T, int H, int G, int D, int Dv, int f32,
+                               hipStream_t s) {
   if (T <= 0) return 0;
   if (Dv > 64 * kMaxSlots || D > 8192 || H % G != 0) return -1;
   const dim3 grid(T, H);
@@ -170,11 +173,11 @@ extern "C" int r32_window_attn(const float* q, const void* k_cache, const void* 
   if (f32)
     window_attn_kernel<float><<<grid, 64, shm, s>>>(q, (const float*)k_cache, (const float*)v_cache, kb_stride, vb_stride,
                                                     block_size, positions, cu_q, n_items, block_tables, bt_width, r1, r2,
-                                                    sink, window, chunk, (float*)out, ldo, H, G, D, Dv);
+                                                    sink, window, chunk, cap, (float*)out, ldo, H, G, D, Dv);
   else
     window_attn_kernel<bf16_t><<<grid, 64, shm, s>>>(q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, kb_stride,
                                                      vb_stride, block_size, positions, cu_q, n_items, block_tables,
-                                                     bt_width, r1, r2, sink, window, chunk, (bf16_t*)out, ldo, H, G, D, Dv);
+                                                     bt_width, r1, r2, sink, window, chunk, cap, (bf16_t*)out, ldo, H, G, D, Dv);
   return (int)hipGetLastError();
 }
 
@@ -216,6 +219,7 @@ struct WAttnMfmaParams {
   const float* sink;  // [H], or null: exp(sink_h) joins the softmax denominator of head h (no key, no value)
   int window;
   int chunk;          // > 0: row i sees only keys of its own chunk, j >= i - i % chunk (besides the window)
+  float cap;          // > 0: scores become cap tanh(score / cap)
   bf16_t* out;
   int ldo, H, G;
 };
@@ -270,6 +274,7 @@ __global__ void __launch_bounds__(256) window_attn_mfma_kernel(const WAttnMfmaPa
   const int w_min = pos0 + 16 * w, w_max = min(pos0 + 16 * w + 15, pos_last);  // this wave's positions
   const int w_lo_min = lo_of(w_min), w_lo_max = lo_of(max(w_max, w_min)), lo_q = lo_of(i_q);  // and their first visible keys
   const bool wave_live = 16 * w < nrows;
+  const float cap_k = p.cap > 0.f ? 2.0f * kLog2e / p.cap : 0.f;
 
   float4v O[NV];
 #pragma unroll
@@ -360,6 +365,10 @@ __global__ void __launch_bounds__(256) window_attn_mfma_kernel(const WAttnMfmaPa
         sacc[sub] = mfma16(a, qhi[kd], sacc[sub]);
         sacc[sub] = mfma16(a, qlo[kd], sacc[sub]);
       }
+    }
+    if (p.cap > 0.f) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) sacc[e >> 2][e & 3] = softcap_f(sacc[e >> 2][e & 3], p.cap, cap_k);
     }
     // every key of the tile visible to every row of the wave: no masks
     const bool inner = kt * 32 + 31 <= w_min && kt * 32 >= w_lo_max && w_max - w_min == 15;
@@ -471,7 +480,7 @@ extern "C" int r32_window_attn_mfma_ok(int D, int Dv) {
 extern "C" int r32_window_attn_mfma(const float* q, const void* k_cache, const void* v_cache, long long kb_stride,
                                     long long vb_stride, int block_size, const int* positions, const int* cu_q,
                                     const int* k_lens, int n_items, int max_q, const int* block_tables, int bt_width,
-                                    const float* bias, const float* sink, int window, int chunk, void* out, int ldo, int H, int G,
+                                    const float* bias, const float* sink, int window, int chunk, float cap, void* out, int ldo, int H, int G,
                                     int D, int Dv, hipStream_t s) {
   if (n_items <= 0 || max_q <= 0) return 0;
   if (!r32_window_attn_mfma_ok(D, Dv) || H % G != 0 || (block_size & (block_size - 1)) != 0) return -1;
@@ -482,7 +491,7 @@ extern "C" int r32_window_attn_mfma(const float* q, const void* k_cache, const v
   for (int b = 0; b < 20; ++b)
     if ((1 << b) == block_size) p.bs_shift = b;
   p.cu_q = cu_q; p.k_lens = k_lens; p.tiles_per_item = (max_q + 63) / 64; p.block_tables = block_tables;
-  p.bt_width = bt_width; p.bias = bias; p.sink = sink; p.window = window; p.chunk = chunk; p.out = (bf16_t*)out; p.ldo = ldo; p.H = H; p.G = G;
+  p.bt_width = bt_width; p.bias = bias; p.sink = sink; p.window = window; p.chunk = chunk; p.cap = cap; p.out = (bf16_t*)out; p.ldo = ldo; p.H = H; p.G = G;
   const dim3 grid(n_items * p.tiles_per_item, H);
   // a workgroup's keys span at most window + 63 positions (from a 32-aligned start: + 31) and never more than the table
   long long span = (long long)window + 63 + 31;

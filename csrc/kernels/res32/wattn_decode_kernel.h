@@ -1,6 +1,6 @@
 // Decode rows of the sliding-window attention (see wattn.hip for the scores, the cache layout and the portion kernel).
 #pragma once
-#include "../common.h"
+#include "elem.h"
 
 using namespace lwc;
 
@@ -31,6 +31,7 @@ struct WAttnDecodeParams {
   const float* bias;       // [H, window], or null: no distance bias
   int window;
   int chunk;               // > 0: the row sees only keys of its own chunk, j >= i - i % chunk (besides the window)
+  float cap;               // > 0: scores become cap tanh(score / cap)
   float* part_o;           // [B, H, S, Dv]
   float* part_ml;          // [B, H, S, 2]
   int H, G, S, keys_per_split;  // keys_per_split: a multiple of 32
@@ -99,6 +100,7 @@ __global__ void __launch_bounds__(64 * NW * NC) window_attn_decode_kernel(const 
 #pragma unroll
   for (int n = 0; n < NVW; ++n) O[n] = float4v{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
+  const float cap_k = p.cap > 0.f ? 2.0f * 1.4426950408889634f / p.cap : 0.f;
   const float* bias_h = p.bias ? p.bias + (size_t)h * p.window : nullptr;  // no table: no distance bias
 
   constexpr bool kStage = NW > 1;
@@ -169,6 +171,10 @@ __global__ void __launch_bounds__(64 * NW * NC) window_attn_decode_kernel(const 
       }
     }
     }  // (scores without the split)
+    if (p.cap > 0.f) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) sacc[e >> 2][e & 3] = softcap_f(sacc[e >> 2][e & 3], p.cap, cap_k);
+    }
     float s[8];
     bool ok[8];
     float mx = -1e30f;

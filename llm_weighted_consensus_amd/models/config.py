@@ -365,12 +365,16 @@ class MerudraConfig:
 class RotarySpec:
     """Rotation by position of the first ``dims`` entries of a head: pair i turns by position * f_i, f_i =
     base^(-2i/dims).  ``scaling`` (factor, original, fast, slow) stretches the slow pairs (frequency blending over a
-    ramp of the pair index) and multiplies the cos / sin tables by 0.1 ln(factor) + 1."""
+    ramp of the pair index) and multiplies the cos / sin tables by 0.1 ln(factor) + 1.  ``bands`` (factor, original, low,
+    high): pairs whose wavelength passes original / low are stretched, those below original / high kept, a blend between."""
     dims: int
     base: float
     scaling: Optional[Tuple[float, float, float, float]] = None   # factor, original, fast, slow
+    bands: Optional[Tuple[float, float, float, float]] = None     # factor, original, low, high
 
     def scaling_dict(self) -> Optional[dict]:
+        if self.bands is not None:
+            return dict(zip(("factor", "original", "low", "high"), self.bands))
         if self.scaling is None:
             return None
         f, o, a, b = self.scaling
@@ -379,6 +383,9 @@ class RotarySpec:
     @classmethod
     def from_dict(cls, r: dict) -> "RotarySpec":
         sc = r.get("scaling")
+        if sc and "high" in sc:
+            return cls(dims=int(r["dims"]), base=float(r["base"]),
+                       bands=(float(sc["factor"]), float(sc["original"]), float(sc["low"]), float(sc["high"])))
         return cls(dims=int(r["dims"]), base=float(r["base"]),
                    scaling=None if not sc else (float(sc["factor"]), float(sc["original"]), float(sc["fast"]),
                                                 float(sc["slow"])))
@@ -388,9 +395,10 @@ class RotarySpec:
 class LatentAttentionSpec:
     """Causal softmax attention whose keys / values pass through a low-rank latent (``kv_rank``), the queries too unless
     ``q_rank`` is 0; per head ``dim`` unrotated and ``rot_dim`` rotated query / key entries (the rotated key part is one
-    vector for all heads, pairs interleaved), values of ``vdim``; a sigmoid output gate.  Whether there is a learned sink
-    per head in the softmax's denominator, and whether the gate is per entry or per head, is the design's.
-    ``kv_from``: the layer whose cached latents and rotated key parts this layer reads instead of caching its own."""
+    vector for all heads), values of ``vdim``.  Whether there is a learned sink per head in the softmax's denominator, a
+    sigmoid gate per entry or per head on the output, and how the rotation pairs its entries, is the design's.
+    ``kv_from``: the layer whose cached latents and rotated key parts this layer reads instead of caching its own.
+    ``window``: a row sees itself and the window - 1 positions before it (None: every earlier one)."""
     heads: int
     dim: int
     rot_dim: int
@@ -400,6 +408,7 @@ class LatentAttentionSpec:
     scale: float
     rot: RotarySpec
     kv_from: Optional[int] = None
+    window: Optional[int] = None
 
     kv_heads = 1   # one cached row (latent + rotated part) serves every head
 
@@ -894,9 +903,149 @@ class GefilixConfig:
         return n
 
 
+# ------------------------------------------------------------------ Semuzen
+@dataclass(frozen=True)
+class CappedAttentionSpec:
+    """Causal softmax attention over grouped heads with capped scores, softcap * tanh(s / softcap) (0: no cap): biases on q,
+    k, v and the output, RMS norms of q and k over their whole projections, rotary positions on the first ``rot.dims``
+    entries of every head (rotate-half pairing), a sigmoid gate per output entry.  ``kv_from``: the layer whose cached keys
+    and values this layer reads instead of projecting its own."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: float
+    rot: RotarySpec
+    kv_from: Optional[int] = None
+
+    @property
+    def nq(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def nk(self) -> int:
+        return self.kv_heads * self.dim
+
+    @property
+    def nv(self) -> int:
+        return self.kv_heads * self.vdim
+
+    @property
+    def no(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class Relu2FfSpec:
+    """Ungated feed-forward W_down relu(W_up h)^2."""
+    ff: int
+
+
+@dataclass(frozen=True)
+class SemuzenLayerSpec:
+    type: str                       # "latent_attention" | "attention"
+    mixer: object                   # LatentAttentionSpec (q_rank 0, a window) | CappedAttentionSpec
+    mlp: Optional[Relu2FfSpec]      # None: no feed-forward in this layer
+
+
+@dataclass(frozen=True)
+class SemuzenConfig:
+    """Semuzen: ``streams`` parallel fp32 residual streams that every sublayer reads through learned weights and mixes
+    anew, an elementwise tanh norm in front of every sublayer, mixers = windowed low-rank attention or capped grouped
+    attention (a layer may read another one's keys and values), ungated relu-squared feed-forwards; a scaled and normed
+    embedding, output weights of their own."""
+    name: str
+    vocab_size: int
+    hidden: int
+    layer_specs: Tuple[SemuzenLayerSpec, ...]
+    norm_eps: float
+    streams: int
+    embed_scale: float
+    bos_token_id: int = 1
+    eos_token_id: int = 2
+
+    architecture = "Semuzen"
+    num_experts = 0   # the engine's expert-parallel planning does not apply
+
+    @property
+    def layers(self) -> int:
+        return len(self.layer_specs)
+
+    @property
+    def heads(self) -> int:
+        return max(L.mixer.heads for L in self.layer_specs)
+
+    @property
+    def kv_heads(self) -> int:
+        return max(L.mixer.kv_heads for L in self.layer_specs)
+
+    @property
+    def head_dim(self) -> int:
+        return max(L.mixer.dim for L in self.layer_specs)
+
+    @classmethod
+    def from_dict(cls, c: dict, name: str = "semuzen") -> "SemuzenConfig":
+        specs = []
+        for i, L in enumerate(c["layers"]):
+            m = L["mixer"]
+            rot = RotarySpec.from_dict(m["rot"])
+            if L["type"] == "latent_attention":
+                mask = m.get("mask")
+                mixer = LatentAttentionSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                                            q_rank=0, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), rot=rot,
+                                            window=int(mask["size"]) if mask else None)
+                if rot.dims != mixer.rot_dim or rot.dims % 2:
+                    raise ValueError("Semuzen: a latent attention layer rotates its whole rot_dim part (an even size)")
+                if mixer.window is not None and mixer.window < 1:
+                    raise ValueError("Semuzen: mask.size must be at least 1")
+            elif L["type"] == "attention":
+                src = m.get("kv_from")
+                mixer = CappedAttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                            scale=float(m["scale"]), softcap=float(m.get("softcap") or 0.0), rot=rot,
+                                            kv_from=None if src is None else int(src))
+                if mixer.heads % mixer.kv_heads:
+                    raise ValueError("Semuzen: heads must be a multiple of kv_heads")
+                if rot.dims % 2 or rot.dims > mixer.dim:
+                    raise ValueError("Semuzen: rot.dims must be even and at most dim")
+                if src is not None:
+                    o = specs[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+                    if (not isinstance(o, CappedAttentionSpec) or o.kv_from is not None
+                            or (o.kv_heads, o.dim, o.vdim) != (mixer.kv_heads, mixer.dim, mixer.vdim)):
+                        raise ValueError("Semuzen: kv_from names an earlier attention layer with projections of its own and the "
+                                         "same kv_heads, dim and vdim")
+            else:
+                raise ValueError(f"Semuzen: unknown mixer type {L['type']!r}")
+            mlp = L.get("mlp")
+            if mlp is not None and mlp.get("kind") != "dense":
+                raise ValueError(f"Semuzen: unknown feed-forward kind {mlp.get('kind')!r}")
+            specs.append(SemuzenLayerSpec(L["type"], mixer, None if mlp is None else Relu2FfSpec(int(mlp["ff"]))))
+        if not specs or int(c["streams"]) < 1:
+            raise ValueError("Semuzen: at least one layer and one stream")
+        return cls(name=name, vocab_size=int(c["vocab"]), hidden=int(c["width"]), layer_specs=tuple(specs),
+                   norm_eps=float(c["norm"]["eps"]), streams=int(c["streams"]), embed_scale=float(c["embedding"]["scale"]))
+
+    def params(self) -> int:
+        d, S = self.hidden, self.streams
+        n = 2 * self.vocab_size * d + 2 * (2 * d + 1)
+        per_sub = 2 * d + 1 + S * S + 2 * S
+        for L in self.layer_specs:
+            m = L.mixer
+            n += per_sub
+            if L.type == "latent_attention":
+                n += d * (m.nq + m.kv_rank + m.rot_dim) + m.kv_rank + m.kv_rank * m.heads * (m.dim + m.vdim) + d * m.nv
+            else:
+                n += (d + 2) * m.nq + 2 * d * m.no + d
+                if m.kv_from is None:
+                    n += (d + 2) * m.nk + (d + 1) * m.nv
+            if L.mlp is not None:
+                n += per_sub + 2 * d * L.mlp.ff
+        return n
+
+
 # config.json "architecture" -> config class of the layer-list decoders
 ARCHITECTURES = {"Madipel": MadipelConfig, "Merudra": MerudraConfig, "Limatar": LimatarConfig, "Rerozen": RerozenConfig,
-                 "Gefilix": GefilixConfig}
+                 "Gefilix": GefilixConfig, "Semuzen": SemuzenConfig}
 
 
 def load_model_config(model_dir) -> object:

@@ -1,5 +1,5 @@
-"""What decoder designs with low-rank ("latent") attention and recurrent layers share: the step functions over the paged
-cache and the state slots, and the attention over cached latents.
+"""What decoder designs with low-rank ("latent") attention share, with recurrent layers or without: the step functions over
+the paged cache and the state slots, and the attention over cached latents (causal, or within a sliding window).
 
 A low-rank attention layer caches ONE row per token for all heads, [latent c | rotated key part], and c again as the value
 row.  Two ways to attend (``LatentDecoder._latent_attention``):
@@ -33,6 +33,15 @@ def up(n: int, m: int) -> int:
     return -(-n // m) * m
 
 
+def adjacent_pairs(w: torch.Tensor, R: int, heads: int = 1) -> torch.Tensor:
+    """Rows of a projection whose last R rows per head are rotated in "rotate half" pairs (i, i + R/2), reordered so that a
+    pair is adjacent (2i, 2i + 1).  Applied to the query and the key side alike it changes no score."""
+    o = w.view(heads, -1, w.shape[-1])
+    n = o.shape[1] - R
+    rot = o[:, n:].view(heads, 2, R // 2, -1).transpose(1, 2).reshape(heads, R, -1)
+    return torch.cat([o[:, :n], rot], 1).reshape(w.shape).contiguous()
+
+
 def core_size(n: int) -> int:
     """The next head size the matrix-core attention kernels are built for (beyond 128: a multiple of 8)."""
     for c in (32, 64, 128):
@@ -53,7 +62,8 @@ class StepAttention:
 
 class LatentDecoder:
     """Base of the designs: subclasses set ``cfg``, ``device``, ``dtype``, ``logit_width``, the weights, and implement
-    ``tensor_shapes``, ``_layer_dims`` (cache rows), ``state_fields``, ``_forward``, ``_gemm_weights`` and ``_head``."""
+    ``tensor_shapes``, ``_layer_dims`` (cache rows), ``_forward``, ``_gemm_weights``, ``_head`` and, with recurrent layers,
+    ``state_fields`` (without: ``has_state = False``, and the step functions take no state)."""
 
     paged_prefill = True      # whole prompts run as one portion over the paged cache (engine._run_prefill)
     supports_cascade = False
@@ -200,12 +210,28 @@ class LatentDecoder:
     def bytes_per_state_slot(self) -> int:
         return RecurrentStatePool.bytes_per_slot(self.state_fields())
 
-    # ------------------------------------------------------------------ attention over cached latents
+    # ------------------------------------------------------------------ attention over the paged cache
     def _no_bias(self, H: int) -> torch.Tensor:
         z = self._zeros_h.get(H)
         if z is None:
             z = self._zeros_h[H] = torch.zeros(H, dtype=torch.float32, device=self.device)
         return z
+
+    def _paged_attention(self, q: torch.Tensor, positions: torch.Tensor, cache: PagedLayerCache, ci: int, plan: StepAttention,
+                         out: torch.Tensor, H: int, G: int, window: Optional[int] = None, cap: float = 0.0,
+                         sink: Optional[torch.Tensor] = None, values_in_keys: bool = False) -> torch.Tensor:
+        """Softmax attention of a step's rows (fp32 ``q`` [n, H * key size]; decode rows first, then portion rows if ``n``
+        reaches them) over cache layer ``ci`` into ``out`` [n, H * value size]."""
+        n, n_dec = q.shape[0], plan.n_dec
+        z, kc, vc, win = self._no_bias(H), cache.k[ci], cache.v[ci], UNBOUNDED if window is None else window
+        if n_dec:
+            res32.window_attn(q[:n_dec], kc, vc, positions[:n_dec], plan.dec_tables, z, z, win, out[:n_dec], H, G, cores=True,
+                              sink=sink, values_in_keys=values_in_keys, cap=cap)
+        if n > n_dec:
+            ch = plan.chunk
+            res32.window_attn(q[n_dec:], kc, vc, positions[n_dec:], ch["block_tables"], z, z, win, out[n_dec:], H, G, cu_q=ch["cu_q"],
+                              k_lens=ch.get("k_lens"), max_q=int(ch.get("max_q", 0)), cores=True, sink=sink, cap=cap)
+        return out
 
     def _latent_attention(self, q: torch.Tensor, x: Dict[str, object], m, ci: int, positions, cache: PagedLayerCache,
                           plan: StepAttention, sink: Optional[torch.Tensor] = None) -> List[Tuple[slice, torch.Tensor]]:
@@ -218,46 +244,45 @@ class LatentDecoder:
         n_dec = plan.n_dec
         wide = T > n_dec and self.expanded_head_sizes(m) is not None and cache.block_size & (cache.block_size - 1) == 0
         n_abs = n_dec if wide else T   # rows that attend over the cached latent rows themselves
-        z, kc, vc = self._no_bias(H), cache.k[ci], cache.v[ci]
         out: List[Tuple[slice, torch.Tensor]] = []
         if n_abs:
             qa, pa = q[:n_abs], positions[:n_abs]
             qn = self._bmm32(qa.view(n_abs, H, D + R)[:, :, :D].transpose(0, 1), x["w_uk"])  # [H, n, C]: keys' up-projection on q
             qf = res32.latent_q_rows(qa, D, R, qn, x["freq"], x["rot_mult"], m.scale, pa, H, Dk).view(n_abs, H * Dk)
             oc = torch.empty(n_abs, H * Cv, dtype=dt, device=self.device)
-            if n_dec:
-                res32.window_attn(qf[:n_dec], kc, vc, pa[:n_dec], plan.dec_tables, z, z, UNBOUNDED, oc[:n_dec], H, 1,
-                                  cores=True, sink=sink, values_in_keys=True)
-            if n_abs > n_dec:
-                ch = plan.chunk
-                res32.window_attn(qf[n_dec:], kc, vc, pa[n_dec:], ch["block_tables"], z, z, UNBOUNDED, oc[n_dec:], H, 1,
-                                  cu_q=ch["cu_q"], k_lens=ch.get("k_lens"), max_q=int(ch.get("max_q", 0)), cores=True,
-                                  sink=sink)
+            self._paged_attention(qf, pa, cache, ci, plan, oc, H, 1, window=m.window, sink=sink, values_in_keys=True)
             o = torch.bmm(oc.view(n_abs, H, Cv)[:, :, :C].transpose(0, 1), x["w_uv_t"])      # [H, n, Dv]
             out.append((slice(0, n_abs), o.transpose(0, 1)))
         if wide:
             out.append((slice(n_dec, T), self._expanded_attention(q[n_dec:], positions[n_dec:], x, m, ci, cache, plan, sink)))
         return out
 
-    def _context_rows(self, plan: StepAttention, bs: int) -> dict:
-        """For the prompt portions of a step: where every token of their sequences (the keys they may see) lies in the
-        paged cache, and a dense page numbering of those tokens, sequence after sequence (built once per step)."""
-        ctx = plan.scratch.get("ctx")
+    def _context_rows(self, plan: StepAttention, bs: int, window: Optional[int] = None) -> dict:
+        """For the prompt portions of a step: where every token that their rows may see lies in the paged cache (the whole
+        sequences, or with ``window`` from the page of the first portion row's first key on), and a dense page numbering of
+        those tokens, sequence after sequence (built once per step and window).  Tables are indexed by position as usual;
+        entries of pages before the first visible key are not read."""
+        ctx = plan.scratch.get(("ctx", window))
         if ctx is None:
             ch = plan.chunk
-            k_lens = np.asarray(ch["lens"][1], dtype=np.int64)
-            pages = -(-k_lens // bs)
-            first = np.concatenate([[0], np.cumsum(pages)])
-            item = np.repeat(np.arange(len(k_lens)), k_lens)
-            pos = np.concatenate([np.arange(n) for n in k_lens]) if len(k_lens) else np.zeros(0, np.int64)
+            q_lens, k_lens = (np.asarray(ch["lens"][i], dtype=np.int64) for i in (0, 1))
+            lo = np.zeros_like(k_lens)
+            if window is not None:   # (the portion kernel walks tiles of 32 keys from a multiple of 32 on)
+                align = max(bs, 32)
+                lo = np.maximum(k_lens - q_lens - window + 1, 0) // align * align
+            skip, last = lo // bs, -(-k_lens // bs)
+            first = np.concatenate([[0], np.cumsum(last - skip)])
+            item = np.repeat(np.arange(len(k_lens)), k_lens - lo)
+            pos = np.concatenate([np.arange(a, n) for a, n in zip(lo, k_lens)]) if len(k_lens) else np.zeros(0, np.int64)
             dev = self.device
             item_d, pos_d = torch.from_numpy(item).to(dev), torch.from_numpy(pos).to(dev)
             blk = ch["block_tables"][item_d, pos_d // bs].long()
-            tables = np.zeros((len(k_lens), max(1, int(pages.max()))), np.int32)
-            for i, n in enumerate(pages):
-                tables[i, :n] = first[i] + np.arange(n)
-            ctx = plan.scratch["ctx"] = {"blk": blk, "off": pos_d % bs, "slots": torch.from_numpy(first[item] * bs + pos).to(dev),
-                                         "tables": torch.from_numpy(tables).to(dev), "pages": int(first[-1])}
+            tables = np.zeros((len(k_lens), max(1, int(last.max()))), np.int32)
+            for i in range(len(k_lens)):
+                tables[i, skip[i]:last[i]] = first[i] + np.arange(last[i] - skip[i])
+            ctx = plan.scratch[("ctx", window)] = {
+                "blk": blk, "off": pos_d % bs, "slots": torch.from_numpy((first[item] - skip[item]) * bs + pos).to(dev),
+                "tables": torch.from_numpy(tables).to(dev), "pages": int(first[-1])}
         return ctx
 
     def _expanded_attention(self, q, positions, x, m, ci: int, cache: PagedLayerCache, plan: StepAttention, sink) -> torch.Tensor:
@@ -266,12 +291,12 @@ class LatentDecoder:
         Tq, bs = q.shape[0], cache.block_size
         C, R, D, H, Dv = m.kv_rank, m.rot_dim, m.dim, m.heads, m.vdim
         dk, dv = self.expanded_head_sizes(m)
-        ctx = self._context_rows(plan, bs)
-        rows = plan.scratch.get(("rows", ci))                                      # [N, row]: latent | rotated part
+        ctx = self._context_rows(plan, bs, m.window)
+        rows = plan.scratch.get(("rows", ci, m.window))                            # [N, row]: latent | rotated part
         if rows is None:   # (a later layer that reads the same cached rows finds them gathered)
-            rows = plan.scratch[("rows", ci)] = cache.k[ci][ctx["blk"], ctx["off"]]
+            rows = plan.scratch[("rows", ci, m.window)] = cache.k[ci][ctx["blk"], ctx["off"]]
         kv = F.linear(rows[:, :C], x["w_ukv"])                                     # [N, H D + H Dv]
-        key = ("pages", H * dk, H * dv)
+        key = ("pages", H * dk, H * dv, ctx["pages"])
         tmp = plan.scratch.get(key)
         if tmp is None:
             tmp = plan.scratch[key] = PagedLayerCache([(H * dk, H * dv)], ctx["pages"], bs, self.device, self.dtype)
@@ -279,14 +304,18 @@ class LatentDecoder:
         qf = res32.latent_q_rows(q, D, R, None, x["freq"], x["rot_mult"], m.scale, positions, H, dk)
         out = torch.empty(Tq, H * dv, dtype=self.dtype, device=self.device)
         ch, z = plan.chunk, self._no_bias(H)
-        res32.window_attn(qf.view(Tq, H * dk), tmp.k[0], tmp.v[0], positions, ctx["tables"], z, z, UNBOUNDED, out, H, H,
+        res32.window_attn(qf.view(Tq, H * dk), tmp.k[0], tmp.v[0], positions, ctx["tables"], z, z,
+                          UNBOUNDED if m.window is None else m.window, out, H, H,
                           cu_q=ch["cu_q"], k_lens=ch["k_lens"], max_q=int(ch["max_q"]), cores=True, sink=sink)
         return out.view(Tq, H, dv)[:, :, :Dv]
 
     # ------------------------------------------------------------------ step functions
-    def _logits(self, x: torch.Tensor, rows: Optional[torch.Tensor], float_logits: bool) -> torch.Tensor:
-        h = res32.rmsnorm_rows(x, self.final_w, self.cfg.norm_eps, self.dtype, rows=rows)
-        lg = self._linear(h, self._head()).float()
+    def _output_rows(self, x, rows: Optional[torch.Tensor]) -> torch.Tensor:
+        """What the output weights read: the output norm of what ``_forward`` returned, optionally of ``rows`` only."""
+        return res32.rmsnorm_rows(x, self.final_w, self.cfg.norm_eps, self.dtype, rows=rows)
+
+    def _logits(self, x, rows: Optional[torch.Tensor], float_logits: bool) -> torch.Tensor:
+        lg = self._linear(self._output_rows(x, rows), self._head()).float()
         if float_logits:
             return lg
         V, Vp = self.cfg.vocab_size, self.logit_width
@@ -302,9 +331,11 @@ class LatentDecoder:
                state_slots: Optional[torch.Tensor] = None) -> torch.Tensor:
         """One decode step for B sequences -> logits [B, V]; device tensors only (hipGraph-capturable).  Row b
         reads table row b and the state slot ``state_slots[b]``; its key range ends at its own position."""
-        if state is None or state_slots is None:
-            raise RuntimeError(f"{self.design}: a decode step needs the recurrent-state pool and the rows' slots")
-        items = res32.StepItems.rows(state_slots, positions)
+        items = None
+        if self.has_state:
+            if state is None or state_slots is None:
+                raise RuntimeError(f"{self.design}: a decode step needs the recurrent-state pool and the rows' slots")
+            items = res32.StepItems.rows(state_slots, positions)
         x = self._forward(tokens, positions, slots, cache, state, items, StepAttention(tokens.shape[0], block_tables, None))
         return self._logits(x, None, float_logits)
 
@@ -315,22 +346,26 @@ class LatentDecoder:
         """ONE forward over [n_dec decode rows || prompt-portion rows]: every projection is one GEMM over both, the
         recurrence walks decode rows and portions alike as items; the attention runs per part over the paged cache
         that this step's rows were just written to.  ``state_slots``: int32, the slot of every decode row, then of
-        every portion.  Logits of ``logit_rows``."""
+        every portion (designs without recurrent layers: no state, no slots).  Logits of ``logit_rows``."""
+        T = tokens.shape[0]
+        items = self._step_items(chunk, T, n_dec, positions, state, state_slots) if self.has_state else None
+        plan = StepAttention(n_dec, dec["block_tables"] if n_dec else None, chunk if T > n_dec else None)
+        keep = logit_rows if n_dec == 0 and self.on_layer is None and 4 * logit_rows.numel() <= T else None
+        x = self._forward(tokens, positions, slots, cache, state, items, plan, keep=keep)
+        return self._logits(x, None if keep is not None else logit_rows, float_logits)
+
+    def _step_items(self, chunk, T: int, n_dec: int, positions, state, state_slots) -> res32.StepItems:
+        """The step's rows grouped by sequence for the recurrent layers: decode rows, then portions."""
         if state is None or state_slots is None:
             raise RuntimeError(f"{self.design}: a step needs the recurrent-state pool and the sequences' slots")
-        T = tokens.shape[0]
         q_lens = list(chunk["lens"][0]) if T > n_dec else []
         cu = np.concatenate([np.arange(n_dec, dtype=np.int64), n_dec + np.concatenate([[0], np.cumsum(q_lens, dtype=np.int64)])])
         if cu[-1] != T or state_slots.numel() != n_dec + len(q_lens):
             raise ValueError(f"{self.design}: rows, portions and state slots disagree")
         row_item = np.concatenate([np.arange(n_dec, dtype=np.int64), n_dec + np.repeat(np.arange(len(q_lens)), q_lens)])
         dev = self.device
-        items = res32.StepItems(torch.from_numpy(row_item.astype(np.int32)).to(dev), torch.from_numpy(cu.astype(np.int32)).to(dev),
-                                state_slots, positions)
-        plan = StepAttention(n_dec, dec["block_tables"] if n_dec else None, chunk if T > n_dec else None)
-        keep = logit_rows if n_dec == 0 and self.on_layer is None and 4 * logit_rows.numel() <= T else None
-        x = self._forward(tokens, positions, slots, cache, state, items, plan, keep=keep)
-        return self._logits(x, None if keep is not None else logit_rows, float_logits)
+        return res32.StepItems(torch.from_numpy(row_item.astype(np.int32)).to(dev), torch.from_numpy(cu.astype(np.int32)).to(dev),
+                               state_slots, positions)
 
     def prefill(self, tokens, positions, slots, cu_seqlens, max_seqlen, last_idx, cache, ctx=None):
         raise RuntimeError(f"{self.design} prefills through forward_mixed over the paged cache (paged_prefill)")

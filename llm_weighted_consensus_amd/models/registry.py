@@ -13,7 +13,7 @@ from typing import Optional
 import torch
 
 from .config import (ARCHITECTURES, DECODERS, GefilixConfig, LimatarConfig, MadipelConfig, MerudraConfig, RerozenConfig,
-                     decoder_config, load_model_config)
+                     SemuzenConfig, decoder_config, load_model_config)
 
 DTYPES = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32, "fp32": torch.float32}
 
@@ -46,6 +46,10 @@ def model_class(cfg):
         from .gefilix import GefilixModel
 
         return GefilixModel
+    if isinstance(cfg, SemuzenConfig):
+        from .semuzen import SemuzenModel
+
+        return SemuzenModel
     if getattr(cfg, "num_experts", 0):
         from .mixtral import MixtralModel
 

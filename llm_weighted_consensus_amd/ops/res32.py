@@ -105,7 +105,8 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
                 block_tables: torch.Tensor, r1: torch.Tensor, r2: torch.Tensor, window: int, out: torch.Tensor,
                 H: int, G: int, cu_q: Optional[torch.Tensor] = None, k_lens: Optional[torch.Tensor] = None,
                 max_q: int = 0, bias: Optional[torch.Tensor] = None, cores: Optional[bool] = None,
-                sink: Optional[torch.Tensor] = None, values_in_keys: bool = False, chunk: int = 0) -> torch.Tensor:
+                sink: Optional[torch.Tensor] = None, values_in_keys: bool = False, chunk: int = 0,
+                cap: float = 0.0) -> torch.Tensor:
     """Sliding-window attention over the paged cache with the bias -r1_h ln(1 + r2_h (i - j)); ``q`` fp32
     [T, H*D] pre-scaled; row t reads table row t (``cu_q`` None) or the item whose ``cu_q`` range holds t.
     Over a bf16 cache whose sizes the matrix-core kernels are built for, prompt portions run on the portion kernel
@@ -117,7 +118,8 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
     (a cached latent that is key and value at once); the decode kernel for one wide row (576 / 512) then takes its
     values from the key rows.
     ``chunk`` > 0: positions are cut into chunks of that many, counted from position 0, and a row sees only keys of its
-    own chunk (j >= i - i % chunk), besides the window."""
+    own chunk (j >= i - i % chunk), besides the window.
+    ``cap`` > 0: a score becomes cap * tanh(score / cap), before the distance bias."""
     K = kernels()
     bs = k_cache.shape[1]
     D, Dv = k_cache.shape[2] // G, v_cache.shape[2] // G
@@ -125,14 +127,14 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
     if cores and cu_q is None and positions.numel() > 0 and K.window_attn_decode_ok(D, Dv, bool(values_in_keys)):
         max_keys = min(int(window), block_tables.shape[1] * k_cache.shape[1], int(chunk) if chunk > 0 else 1 << 30)
         K.window_attn_decode(q, k_cache, v_cache, positions, block_tables, bias, int(window), max_keys, out, int(H), int(G),
-                             sink, bool(values_in_keys), int(chunk))
+                             sink, bool(values_in_keys), int(chunk), float(cap))
         return out
     if cores and cu_q is not None and k_lens is not None and max_q > 0 and K.window_attn_mfma_ok(D, Dv):
         K.window_attn_mfma(q, k_cache, v_cache, positions, cu_q, k_lens, int(max_q), block_tables, bias, int(window), out,
-                           int(H), int(G), sink, int(chunk))
+                           int(H), int(G), sink, int(chunk), float(cap))
         return out
     K.window_attn(q, k_cache, v_cache, positions, cu_q, block_tables, r1, r2, int(window), out, int(H), int(G), sink,
-                  int(chunk))
+                  int(chunk), float(cap))
     return out
 
 
@@ -307,11 +309,18 @@ def rope_frequencies(dims: int, base: float, scaling: Optional[dict] = None, dev
     """(f fp32 [dims / 2], m): the rotation frequencies base^(-2i/dims) and the multiplier of the cos / sin tables.
     ``scaling`` = {factor, original, fast, slow} blends f_i with f_i / factor over a linear ramp of the pair index i
     between the pairs that turn ``fast`` and ``slow`` times within ``original`` positions, and sets
-    m = 0.1 ln(factor) + 1.  Computed in float64, rounded once."""
+    m = 0.1 ln(factor) + 1.  ``scaling`` = {factor, original, low, high}: by wavelength l = 2 pi / f, f_i stays where l <
+    original / high, becomes f_i / factor where l > original / low, and between the two is blended by the share
+    s = (original / l - low) / (high - low) of the unscaled one (m = 1).  Computed in float64, rounded once."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = float(base) ** (-2.0 * i / dims)
     m = 1.0
-    if scaling:
+    if scaling and "high" in scaling:
+        factor, orig, low, high = (float(scaling[k]) for k in ("factor", "original", "low", "high"))
+        turns = orig * f / (2.0 * math.pi)   # original / wavelength
+        s = ((turns - low) / max(high - low, 1e-30)).clamp(0.0, 1.0)
+        f = torch.where(turns > high, f, torch.where(turns < low, f / factor, (1.0 - s) * f / factor + s * f))
+    elif scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
 
         def pair_of(turns: float) -> float:
@@ -350,8 +359,9 @@ def latent_q_rows(q: torch.Tensor, D: int, R: int, qn: Optional[torch.Tensor], f
 
 
 def head_gate_rows(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
-    """out[t, h Dv + i] = o[t, h, i] * sigmoid(gate[t, h]); ``o`` [T, H, Dv] of any row and head strides (a batched product
-    as it lies, padded heads), ``gate`` [T, H] (a column slice is fine)."""
+    """out[t, h Dv + i] = o[t, h, i] * sigmoid(gate[t, h]) (``gate`` [T, H]) or * sigmoid(gate[t, h Dv + i]) (``gate``
+    [T, H Dv]; column slices are fine); ``o`` [T, H, Dv] of any row and head strides (a batched product as it lies, padded
+    heads)."""
     kernels().head_gate_rows(o, gate, out)
     return out
 
@@ -404,7 +414,15 @@ def gelu(z: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """z / 2 (1 + erf(z / sqrt 2)); ``z`` and ``out`` may be column slices of row-dense buffers."""
     if out is None:
         out = torch.empty(z.shape[0], z.shape[1], dtype=z.dtype, device=z.device)
-    kernels().gelu(z, out)
+    kernels().act(z, out, 0)
+    return out
+
+
+def relu2(z: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """max(z, 0)^2; ``z`` and ``out`` may be column slices of row-dense buffers."""
+    if out is None:
+        out = torch.empty(z.shape[0], z.shape[1], dtype=z.dtype, device=z.device)
+    kernels().act(z, out, 1)
     return out
 
 
@@ -423,6 +441,22 @@ def rot_kv_write(src: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor
     kernels().rot_kv_write(src, wq, wk, freq, float(mult), int(rot_dims), vfreq, positions, slots, q_out, k_cache, v_cache,
                            int(H), int(G), float(eps), float(scale))
     return q_out
+
+
+def norm_rot_kv_write(src: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, H: int, D: int, Dk: int, scale: float,
+                      eps: float = 0.0, wq: Optional[torch.Tensor] = None, wk: Optional[torch.Tensor] = None,
+                      bias: Optional[torch.Tensor] = None, rot_dims: int = 0, freq: Optional[torch.Tensor] = None, mult: float = 1.0,
+                      k_cache: Optional[torch.Tensor] = None, v_cache: Optional[torch.Tensor] = None, G: int = 0,
+                      Dv: int = 0) -> torch.Tensor:
+    """:func:`rot_kv_write` for layers whose q and k are RMS-normed over their whole projections: ``src`` rows [q (H D) |
+    k (G D) | v (G Dv)] plus ``bias`` (fp32 per column); q / rms(q) * wq (fp32 [H D]) and k / rms(k) * wk, then the rotation of
+    the first ``rot_dims`` entries of every head; q times ``scale`` -> fp32 [T, H, Dk] (returned), k and v -> the paged cache
+    at ``slots`` (-1: no write).  Heads are padded with zeros to ``Dk`` and to the cache's value size.  ``G`` = 0 and no
+    caches: rows of q only (a layer that reads another layer's keys and values)."""
+    q = torch.empty(src.shape[0], H, Dk, dtype=torch.float32, device=src.device)
+    kernels().norm_rot_kv_write(src, bias, wq, wk, freq, float(mult), int(rot_dims), positions, slots, q, k_cache, v_cache, int(H),
+                                int(G), int(D), int(Dv), float(eps), float(scale))
+    return q
 
 
 def head_gate_unrotate(o: torch.Tensor, out: torch.Tensor, positions: torch.Tensor, H: int, gate: Optional[torch.Tensor] = None,
@@ -460,3 +494,37 @@ def channel_decay_rule(src: torch.Tensor, z: torch.Tensor, state: torch.Tensor, 
     kernels().chan_rule(src, qkv, z, zb, A_log, 1.0 / float(tau), beta, state, items.cu, items.slots, items.positions, out,
                         int(H), int(G), bool(unit), bool(delta))
     return out
+
+
+# ------------------------------------------------------------------ parallel residual streams, bounded norms
+class Dyt:
+    """Parameters of the elementwise norm tanh(a x) * w + b (a: a number, w and b fp32 [d])."""
+
+    def __init__(self, a: float, w: torch.Tensor, b: torch.Tensor):
+        self.a, self.w, self.b = float(a), w, b
+
+
+def hyper_coef(mix: torch.Tensor, out: torch.Tensor, w_in: torch.Tensor) -> torch.Tensor:
+    """The coefficients of one :func:`hyper_step`: mix [S, S] (from, to), out [S], and the following reader's in [S]."""
+    return torch.cat([mix.reshape(-1), out, w_in]).to(torch.float32).contiguous()
+
+
+def embed_streams(table: torch.Tensor, tokens: torch.Tensor, scale: float, norm: Dyt, w_in: torch.Tensor, nxt: Dyt):
+    """(X, h): every stream X[s] (fp32 [S, T, d]) = norm(table[tokens] * scale), h = nxt(sum_s w_in[s] X[s]) in the table's
+    dtype."""
+    T, d = tokens.numel(), table.shape[1]
+    X = torch.empty(w_in.numel(), T, d, dtype=torch.float32, device=table.device)
+    h = torch.empty(T, d, dtype=table.dtype, device=table.device)
+    kernels().embed_streams(table, tokens, float(scale), norm.a, norm.w, norm.b, w_in, nxt.a, nxt.w, nxt.b, X, h)
+    return X, h
+
+
+def hyper_step(X: torch.Tensor, y: torch.Tensor, coef: torch.Tensor, nxt: Dyt, dtype, bias: Optional[torch.Tensor] = None,
+               rows: Optional[torch.Tensor] = None, write: bool = True) -> torch.Tensor:
+    """A sublayer's result y (plus ``bias`` per column) into the streams X (fp32 [S, T, d], in place with ``write``):
+    X'_t = sum_s mix[s, t] X_s + out[t] y; returns h = nxt(sum_t in[t] X'_t) as ``dtype`` rows.  ``coef``:
+    :func:`hyper_coef`.  ``rows`` (int64, needs write=False): only these rows of X and y."""
+    n = X.shape[1] if rows is None else rows.numel()
+    h = torch.empty(n, X.shape[2], dtype=dtype, device=X.device)
+    kernels().hyper_step(X, y, bias, coef, nxt.a, nxt.w, nxt.b, h, rows, bool(write))
+    return h
