@@ -3,7 +3,7 @@
 
     python bench.py --compare-decoders [--sizes small,8b-layer] [--compare-layers 4]
 
-Designs: ``madipel``, ``llama``, ``merudra``, ``mixtral``, ``limatar``, ``rerozen``, ``gefilix`` (``--designs merudra,mixtral`` puts Merudra
+Designs: ``madipel``, ``llama``, ``merudra``, ``mixtral``, ``limatar``, ``rerozen``, ``gefilix``, ``semuzen`` (``--designs merudra,mixtral`` puts Merudra
 beside the closest existing decoder, the routed-experts Mixtral: 8 experts, 2 per token, the same active feed-forward
 width; Merudra's layers alternate attention and gated delta rule mixers and add 2 identity experts.
 ``--designs limatar,merudra`` puts Limatar beside Merudra, the closest decoder with paged attention AND recurrent
@@ -16,6 +16,10 @@ attention AND a half-size channel-decay linear attention side by side, and a den
 rows and a fixed-decay recurrence over an fp32 stream): Gefilix's layers alternate low-rank attention, of which every
 second one reads the latents of the one before, and lightning attention, grouped sigmoid-routed clamped experts with a
 gated shared expert and the dense gelu unit).
+``--designs semuzen,madipel`` puts Semuzen beside Madipel, the closest decoder (windowed paged attention without recurrent
+state and an ungated feed-forward of two matrices over an fp32 stream): Semuzen's layers alternate capped grouped attention,
+of which every second one reads the keys and values of the one before, and windowed low-rank attention, over two residual
+streams.
 
 For each size a Madipel model (parallel layers, windowed attention with distance bias, xIELU feed-forward, fp32
 residual) and the closest existing decoder (Llama: sequential layers, causal GQA attention with RoPE, SwiGLU) are
@@ -159,6 +163,32 @@ def _gefilix(size: dict, layers: int, device, seed: int, experts: int = 8, top: 
     return GefilixModel(cfg, device=device, seed=seed)
 
 
+def _semuzen(size: dict, layers: int, device, seed: int, pattern: str = "al", window: int = 1024, streams: int = 2):
+    """Capped grouped attention and windowed low-rank attention alternating (``pattern``: a / l per layer, repeated; the other
+    designs' second letters mean l); every second attention layer reads the keys and values of the one before.  Heads and head
+    size as in the other designs, latents as in ``_limatar``, windows of ``window`` positions; the ungated feed-forward's two
+    matrices get 1.5x the gated designs' inner width (equal parameters)."""
+    from llm_weighted_consensus_amd.models.config import SemuzenConfig
+    from llm_weighted_consensus_amd.models.semuzen import SemuzenModel
+
+    H, G, D, d = size["heads"], size["kv_heads"], size["head_dim"], size["width"]
+    mlp = {"kind": "dense", "ff": 3 * size["ffn"] // 2}
+    att = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 50.0,
+           "rot": {"base": 5e5, "dims": D, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 1024}}}
+    lat = {"heads": H, "dim": D, "rot_dim": D // 2, "vdim": D, "kv_rank": 4 * D, "scale": (D + D // 2) ** -0.5, "mask": {"size": window},
+           "rot": {"base": 10000.0, "dims": D // 2, "scaling": {"factor": 4.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}
+    specs, own = [], None
+    for i in range(layers):
+        if pattern[i % len(pattern)] == "a":
+            specs.append({"type": "attention", "mixer": att if own is None else dict(att, kv_from=own), "mlp": mlp})
+            own = i if own is None else None
+        else:
+            specs.append({"type": "latent_attention", "mixer": lat, "mlp": mlp})
+    cfg = SemuzenConfig.from_dict({"architecture": "Semuzen", "embedding": {"scale": 1.0}, "layers": specs, "norm": {"eps": 1e-6},
+                                   "streams": streams, "vocab": size["vocab"], "width": d}, name="semuzen-bench")
+    return SemuzenModel(cfg, device=device, seed=seed)
+
+
 def _mixtral(size: dict, layers: int, max_pos: int, device, seed: int, experts: int = 8, top: int = 2):
     from llm_weighted_consensus_amd.models.config import DecoderConfig
     from llm_weighted_consensus_amd.models.mixtral import MixtralModel
@@ -223,6 +253,8 @@ def run(sizes: str = "small,8b-layer", layers: int = 4, prompt_len: int = 2048, 
                 model = _rerozen(size, layers, dev, 3, pattern=pattern)
             elif design == "gefilix":
                 model = _gefilix(size, layers, dev, 3, pattern=pattern)
+            elif design == "semuzen":
+                model = _semuzen(size, layers, dev, 3, pattern=pattern)
             elif design == "limatar":
                 model = _limatar(size, layers, dev, 3, pattern=pattern)
             elif design == "mixtral":
@@ -239,7 +271,7 @@ def run(sizes: str = "small,8b-layer", layers: int = 4, prompt_len: int = 2048, 
             print(json.dumps(line), flush=True)
             summary.setdefault(name, {})[design] = r
     for a, b in (("madipel", "llama"), ("merudra", "mixtral"), ("merudra", "madipel"), ("limatar", "merudra"), ("rerozen", "merudra"),
-                 ("gefilix", "limatar")):
+                 ("gefilix", "limatar"), ("semuzen", "madipel"), ("semuzen", "gefilix")):
         out = {}
         for name, d in summary.items():
             if a in d and b in d:
