@@ -72,8 +72,8 @@ int r32_act(const void*, int, void*, int, int, int, int, int, hipStream_t);
 int r32_hyper_max_streams();
 int r32_embed_streams(const void*, const int*, int, float, float, const float*, const float*, const float*, int, float, const float*,
                       const float*, float*, void*, int, int, int, hipStream_t);
-int r32_hyper_step(float*, long long, int, const void*, int, const float*, const float*, float, const float*, const float*, void*,
-                   const long long*, int, int, int, int, hipStream_t);
+int r32_hyper_step(float*, long long, int, const void*, int, int, long long, const float*, const float*, float, const float*,
+                   const float*, void*, const long long*, int, int, int, int, hipStream_t);
 int r32_norm_rot_kv_write(const void*, int, const float*, const float*, const float*, const float*, float, int, const int*,
                           const int*, float*, void*, void*, long long, long long, int, int, int, int, int, int, int, int, float,
                           float, int, hipStream_t);
@@ -315,10 +315,11 @@ void window_attn_mfma(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions
 }
 
 // One new token per sequence on the matrix cores (bf16 caches): row b reads table row b, its key range ends at
-// positions[b].  max_keys: a host-side upper bound of the keys a row sees (min(window, longest context)).
+// positions[b].  max_keys: a host-side upper bound of the keys a row sees (min(window, longest context)).  splits: key
+// ranges per row, 0: by the sizes.
 void window_attn_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positions, Tensor block_tables,
                         c10::optional<Tensor> bias, int64_t window, int64_t max_keys, Tensor out, int64_t H, int64_t G,
-                        c10::optional<Tensor> sink, bool values_in_keys, int64_t chunk, double cap) {
+                        c10::optional<Tensor> sink, bool values_in_keys, int64_t chunk, double cap, int64_t splits) {
   want(q, torch::kFloat32, "window_attn_decode q");
   want(positions, torch::kInt32, "window_attn_decode positions");
   want(block_tables, torch::kInt32, "window_attn_decode block_tables");
@@ -338,7 +339,8 @@ void window_attn_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor positio
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) >= B && q.numel() == (int64_t)B * H * D && out.size(0) == B &&
                   out.size(1) == H * Dv && window >= 1 && max_keys >= 1 && (!bias.has_value() || bias->numel() == H * window),
               "window_attn_decode: shapes disagree");
-  const int S = r32_window_attn_decode_splits(B, (int)G, (int)(H / G), (int)max_keys, D);
+  TORCH_CHECK(splits >= 0 && splits <= 64, "window_attn_decode: splits");
+  const int S = splits > 0 ? (int)splits : r32_window_attn_decode_splits(B, (int)G, (int)(H / G), (int)max_keys, D);
   auto part = torch::empty({(int64_t)B * H * S * (Dv + 2)}, q.options());
   float* po = part.data_ptr<float>();
   done(r32_window_attn_decode(q.data_ptr<float>(), k_cache.data_ptr(), v_cache.data_ptr(), (long long)k_cache.stride(0),
@@ -978,13 +980,16 @@ void embed_streams(Tensor table, Tensor tokens, double scale, double ae, Tensor 
 }
 
 // X fp32 [S, T, d]: X'_t = sum_s mix[s][t] X_s + out[t] (y + bias) (stored when write), h = dyt(sum_t in[t] X'_t); coef fp32
-// [S S + 2 S] = mix | out | in; y [T, d]; rows (int64, not with write): only these rows, h [len(rows), d]
+// [S S + 2 S] = mix | out | in; y [T, d] or planes [P, T, d] whose sum is the result; rows (int64, not with write): only these rows, h [len(rows), d]
 void hyper_step(Tensor X, Tensor y, c10::optional<Tensor> bias, Tensor coef, double a, Tensor w, Tensor b, Tensor h,
                 c10::optional<Tensor> rows, bool write) {
   want(X, torch::kFloat32, "hyper_step X");
   want(coef, torch::kFloat32, "hyper_step coef");
   const int fy = act_f32(y, "hyper_step y"), fh = act_f32(h, "hyper_step h");
-  const int ldy = row_stride(y, "hyper_step y");
+  TORCH_CHECK(y.dim() == 2 || (y.dim() == 3 && y.is_contiguous() && y.size(0) >= 1), "hyper_step: y [T, d] or planes [P, T, d]");
+  const int parts = y.dim() == 3 ? (int)y.size(0) : 1;
+  const long long ypart = y.dim() == 3 ? (long long)y.stride(0) : 0;
+  const int ldy = row_stride(y.dim() == 3 ? y.select(0, 0) : y, "hyper_step y");
   TORCH_CHECK(X.dim() == 3 && h.dim() == 2 && h.is_contiguous(), "hyper_step: X [S, T, d], h [n, d]");
   const int S = (int)X.size(0), T = (int)X.size(1), d = (int)X.size(2);
   const long long* rp = nullptr;
@@ -995,9 +1000,9 @@ void hyper_step(Tensor X, Tensor y, c10::optional<Tensor> bias, Tensor coef, dou
     n = (int)rows->numel();
     rp = (const long long*)rows->data_ptr<int64_t>();
   }
-  TORCH_CHECK(S >= 1 && S <= r32_hyper_max_streams() && coef.numel() == (int64_t)S * S + 2 * S && y.size(0) == T && y.size(1) == d &&
+  TORCH_CHECK(S >= 1 && S <= r32_hyper_max_streams() && coef.numel() == (int64_t)S * S + 2 * S && y.size(-2) == T && y.size(-1) == d &&
                   h.size(0) == n && h.size(1) == d, "hyper_step: shapes disagree");
-  done(r32_hyper_step(X.data_ptr<float>(), (long long)T * d, S, y.data_ptr(), ldy, opt_f32(bias, d, "hyper_step bias"),
+  done(r32_hyper_step(X.data_ptr<float>(), (long long)T * d, S, y.data_ptr(), ldy, parts, ypart, opt_f32(bias, d, "hyper_step bias"),
                       coef.data_ptr<float>(), (float)a, opt_f32(w, d, "hyper_step w"), opt_f32(b, d, "hyper_step b"), h.data_ptr(), rp,
                       n, d, write ? 1 : 0, fy | (fh << 1), stream()), "hyper_step");
 }

@@ -31,8 +31,9 @@ struct HyperParams {
   float* X;             // [S, T, d]
   long long plane;      // T * d
   int S;
-  const void* y;        // [T, d]
-  int ldy;
+  const void* y;        // [T, d], or `parts` such planes whose sum is the result (the partial products of a split GEMM)
+  int ldy, parts;
+  long long ypart;      // between the planes
   const float* bias;    // [d] or null
   const float* coef;    // [S*S | S | S]
   float a;
@@ -57,7 +58,8 @@ __global__ void __launch_bounds__(256) hyper_step_vec_kernel(const HyperParams p
   for (int r = blockIdx.y; r < p.n; r += gridDim.y) {
     const long long t = p.rows ? p.rows[r] : r;
     float* xr = p.X + t * p.d + c;
-    const float4v y = Vec4<YT>::ld((const YT*)p.y + t * p.ldy + c) + bias;
+    float4v y = Vec4<YT>::ld((const YT*)p.y + t * p.ldy + c) + bias;
+    for (int k = 1; k < p.parts; ++k) y += Vec4<YT>::ld((const YT*)p.y + k * p.ypart + t * p.ldy + c);
     float4v x[NS];
 #pragma unroll
     for (int s = 0; s < NS; ++s)
@@ -89,7 +91,8 @@ __global__ void __launch_bounds__(256) hyper_step_kernel(const HyperParams p) {
   for (int r = blockIdx.y; r < p.n; r += gridDim.y) {
     const long long t = p.rows ? p.rows[r] : r;
     float* xr = p.X + t * p.d + c;
-    const float y = Elem<YT>::ld((const YT*)p.y + t * p.ldy + c) + (p.bias ? p.bias[c] : 0.f);
+    float y = Elem<YT>::ld((const YT*)p.y + t * p.ldy + c) + (p.bias ? p.bias[c] : 0.f);
+    for (int k = 1; k < p.parts; ++k) y += Elem<YT>::ld((const YT*)p.y + k * p.ypart + t * p.ldy + c);
     float x[NS];
 #pragma unroll
     for (int s = 0; s < NS; ++s) x[s] = s < S ? xr[s * p.plane] : 0.f;
@@ -122,7 +125,7 @@ __global__ void __launch_bounds__(256) embed_streams_kernel(const TT* __restrict
   const long long plane = (long long)T * d;
   float g = 0.f;
   for (int s = 0; s < S; ++s) g += in[s];
-  for (int i = threadIdx.x; i < d; i += blockDim.x) {
+  for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < d; i += gridDim.y * blockDim.x) {
     const float x = dyt1<float>(Elem<TT>::ld(row + i) * scale, ae, we[i], be[i]);
     for (int s = 0; s < S; ++s) X[s * plane + (size_t)t * d + i] = x;
     Elem<AT>::st(h + (size_t)t * d + i, dyt1<AT>(x * g, a, w[i], b[i]));
@@ -165,11 +168,13 @@ extern "C" int r32_embed_streams(const void* table, const int* tokens, int vocab
                                  void* h, int T, int d, int io, hipStream_t s) {
   if (T <= 0) return 0;
   if (S < 1 || S > r32_hyper_max_streams()) return -1;
+  const int parts = (d + 255) / 256;
+  const dim3 grid(T, T >= 1024 ? 1 : (parts < 16 ? parts : 16));  // few rows: several workgroups per row
   if (io == 3)
-    embed_streams_kernel<float, float><<<T, 256, 0, s>>>((const float*)table, tokens, vocab, scale, ae, we, be, in, S, a, w, b, X,
+    embed_streams_kernel<float, float><<<grid, 256, 0, s>>>((const float*)table, tokens, vocab, scale, ae, we, be, in, S, a, w, b, X,
                                                          (float*)h, T, d);
   else if (io == 0)
-    embed_streams_kernel<bf16_t, bf16_t><<<T, 256, 0, s>>>((const bf16_t*)table, tokens, vocab, scale, ae, we, be, in, S, a, w, b,
+    embed_streams_kernel<bf16_t, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)table, tokens, vocab, scale, ae, we, be, in, S, a, w, b,
                                                            X, (bf16_t*)h, T, d);
   else
     return -1;
@@ -178,16 +183,16 @@ extern "C" int r32_embed_streams(const void* table, const int* tokens, int vocab
 }
 
 // io: bit 0 = y fp32 (else bf16), bit 1 = h fp32 (else bf16)
-extern "C" int r32_hyper_step(float* X, long long plane, int S, const void* y, int ldy, const float* bias, const float* coef, float a,
-                              const float* w, const float* b, void* h, const long long* rows, int n, int d, int write, int io,
+extern "C" int r32_hyper_step(float* X, long long plane, int S, const void* y, int ldy, int parts, long long ypart, const float* bias,
+                              const float* coef, float a, const float* w, const float* b, void* h, const long long* rows, int n, int d, int write, int io,
                               hipStream_t s) {
   if (n <= 0) return 0;
-  if (S < 1 || S > r32_hyper_max_streams() || (write && rows)) return -1;
+  if (S < 1 || S > r32_hyper_max_streams() || (write && rows) || parts < 1) return -1;
   HyperParams p;
-  p.X = X; p.plane = plane; p.S = S; p.y = y; p.ldy = ldy; p.bias = bias; p.coef = coef; p.a = a; p.w = w; p.b = b; p.h = h;
+  p.X = X; p.plane = plane; p.S = S; p.y = y; p.ldy = ldy; p.parts = parts; p.ypart = ypart; p.bias = bias; p.coef = coef; p.a = a; p.w = w; p.b = b; p.h = h;
   p.rows = rows; p.n = n; p.d = d; p.write = write;
   const bool yf = io & 1, hf = io & 2;
-  const bool vec = d % 4 == 0 && ldy % 4 == 0 && plane % 4 == 0 && aligned_to(X, 16) && aligned_to(y, yf ? 16 : 8) &&
+  const bool vec = d % 4 == 0 && ldy % 4 == 0 && ypart % 4 == 0 && plane % 4 == 0 && aligned_to(X, 16) && aligned_to(y, yf ? 16 : 8) &&
                    aligned_to(bias, 16) && aligned_to(w, 16) && aligned_to(b, 16) && aligned_to(h, hf ? 16 : 8);
   if (yf && hf) launch_hyper<float, float>(p, vec, s);
   else if (!yf && !hf) launch_hyper<bf16_t, bf16_t>(p, vec, s);

@@ -102,6 +102,41 @@ latent_q_rows_kernel(const AT* __restrict__ q, int ldq, int D, int R, const floa
   }
 }
 
+// Four entries per thread: D, R, C, Dk and every base multiples of four; the row's angles are formed once for all heads.
+// blockIdx.y: parts of a row (few rows leave most of the chip idle otherwise).
+template <typename AT>
+__global__ void __launch_bounds__(256)
+latent_q_rows_vec_kernel(const AT* __restrict__ q, int ldq, int D, int R, const float* __restrict__ qn, int C,
+                         const float* __restrict__ freq, float mult, float scale, const int* __restrict__ positions,
+                         float* __restrict__ out, int H, int Dk, int T) {
+  extern __shared__ __attribute__((aligned(16))) float ang[];  // [R]: cos, sin of pair 0, of pair 1, ...
+  const int t = blockIdx.x;
+  const float p = (float)positions[t];
+  for (int i = threadIdx.x; i < R / 2; i += blockDim.x) {
+    float sn, cs;
+    sincosf(p * freq[i], &sn, &cs);
+    ang[2 * i] = cs * (mult * scale);
+    ang[2 * i + 1] = sn * (mult * scale);
+  }
+  __syncthreads();
+  const int k4 = Dk >> 2;
+  float* o = out + (size_t)t * H * Dk;
+  const AT* qr = q + (size_t)t * ldq;
+  for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < H * k4; e += gridDim.y * blockDim.x) {
+    const int h = e / k4, i = (e - h * k4) * 4;
+    float4v x = float4v{0.f, 0.f, 0.f, 0.f};
+    if (i < C) {
+      // without qn the unrotated part is the row's own (C == D then)
+      x = (qn ? Vec4<float>::ld(qn + ((size_t)h * T + t) * C + i) : Vec4<AT>::ld(qr + (size_t)h * (D + R) + i)) * scale;
+    } else if (i < C + R) {
+      const int r = i - C;
+      const float4v u = Vec4<AT>::ld(qr + (size_t)h * (D + R) + D + r), a = Vec4<float>::ld(ang + r);
+      x = float4v{u[0] * a[0] - u[1] * a[1], u[1] * a[0] + u[0] * a[1], u[2] * a[2] - u[3] * a[3], u[3] * a[2] + u[2] * a[3]};
+    }
+    Vec4<float>::st(o + 4 * (size_t)e, x);
+  }
+}
+
 // One workgroup per token: key rows [H][dk] = [kv key of the head (D) | the token's rotated part (R) | 0], value rows
 // [H][dv] = [kv value | 0] in the 4-token interleaved layout.
 template <typename AT>
@@ -234,6 +269,18 @@ extern "C" int r32_latent_q_rows(const void* q, int ldq, int D, int R, const flo
                                  hipStream_t s) {
   if (T <= 0) return 0;
   if (R % 2 != 0 || Dk < C + R) return -1;
+  if (D % 4 == 0 && R % 4 == 0 && C % 4 == 0 && Dk % 4 == 0 && ldq % 4 == 0 && R <= 4096 && aligned_to(q, f32 ? 16 : 8) &&
+      aligned_to(qn, 16) && aligned_to(out, 16)) {
+    const int parts = (H * (Dk / 4) + 255) / 256;
+    const dim3 grid(T, T >= 1024 ? 1 : (parts < 16 ? parts : 16));
+    const size_t shm = (size_t)(R ? R : 4) * sizeof(float);
+    if (f32)
+      latent_q_rows_vec_kernel<float><<<grid, 256, shm, s>>>((const float*)q, ldq, D, R, qn, C, freq, mult, scale, positions, out, H, Dk, T);
+    else
+      latent_q_rows_vec_kernel<bf16_t><<<grid, 256, shm, s>>>((const bf16_t*)q, ldq, D, R, qn, C, freq, mult, scale, positions, out, H, Dk, T);
+    LWC_CHECK_LAUNCH();
+    return 0;
+  }
   if (f32)
     latent_q_rows_kernel<float><<<T, 256, 0, s>>>((const float*)q, ldq, D, R, qn, C, freq, mult, scale, positions, out, H, Dk, T);
   else

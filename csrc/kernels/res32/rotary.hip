@@ -261,7 +261,7 @@ __global__ void __launch_bounds__(256) norm_rot_kv_write_kernel(const NormRotPar
 
 // D, Dv, Dk, Dvp multiples of four, rd a multiple of eight, every base a multiple of four entries
 template <typename IT, typename CT>
-__global__ void __launch_bounds__(256) norm_rot_kv_write_vec_kernel(const NormRotParams p) {
+__global__ void __launch_bounds__(1024) norm_rot_kv_write_vec_kernel(const NormRotParams p) {
   extern __shared__ __attribute__((aligned(16))) float tab[];  // [rd] angles
   __shared__ float scratch[16];
   const int t = blockIdx.x, H = p.H, G = p.G, D = p.D, Dv = p.Dv, half = p.rd >> 1;
@@ -443,8 +443,9 @@ extern "C" int r32_norm_rot_kv_write(const void* src, int lds, const float* bias
                    aligned_to(src, ib) && aligned_to(k_cache, cb) && aligned_to(q_out, 16) && aligned_to(bias, 16) &&
                    aligned_to(wq, 16) && aligned_to(wk, 16);
   const size_t shm = (size_t)(rd ? rd : 4) * sizeof(float);
+  const int threads = T >= 1024 || H * Dk <= 1024 ? 256 : 1024;  // few long rows: more waves per row
 #define LWC_NRK(IT, CT)                                          \
-  if (vec) norm_rot_kv_write_vec_kernel<IT, CT><<<T, 256, shm, s>>>(p); \
+  if (vec) norm_rot_kv_write_vec_kernel<IT, CT><<<T, threads, shm, s>>>(p); \
   else norm_rot_kv_write_kernel<IT, CT><<<T, 256, 0, s>>>(p)
   if (io == 3) {
     LWC_NRK(float, float);

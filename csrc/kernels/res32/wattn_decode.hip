@@ -49,13 +49,14 @@ int launch_decode_nv(const WAttnDecodeParams& p, int nv, dim3 grid, hipStream_t 
 // Splits for a decode step of B sequences whose windows hold at most max_keys keys: about 2048 waves (two per SIMD),
 // at least 64 keys each.  Measured at 64 sequences x 8 kv heads x 2048 keys of 128: 3 splits 150 us, 4 splits
 // (2048 waves) 130 us, 8 splits 155 us, 16 splits 146 us (shorter key runs per wave, larger partials to merge).
-// Wide rows (D = 320, 576): workgroups of four or eight waves, about 512 of them, at least 128 keys each (their partials
-// are large).
+// Wide rows (D = 320, 576): workgroups of four waves, about 512 of them, or of eight (more than 16 heads), at most 256 of them
+// (one per CU: at 64 sequences x 32 heads x 576 / 512 over 2048 keys 4 splits take 105 us where 8 take 139 us), at least 128
+// keys each (their partials are large).
 extern "C" int r32_window_attn_decode_splits(int B, int G, int Hg, int max_keys, int D) {
   const bool wide = D > 192;
   const int chunks = (Hg + 15) / 16;
   const int waves = B * G * (wide && chunks > 1 ? (chunks + 1) / 2 : chunks);  // wide rows: workgroups
-  int s = ((wide ? 512 : 2048) + waves - 1) / waves;
+  int s = wide && chunks > 1 ? 256 / waves : ((wide ? 512 : 2048) + waves - 1) / waves;
   const int by_keys = wide ? (max_keys + 32 + 127) / 128 : (max_keys + 32 + 63) / 64;
   if (s > by_keys) s = by_keys;
   if (s > 64) s = 64;

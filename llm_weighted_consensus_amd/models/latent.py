@@ -88,6 +88,8 @@ class LatentDecoder:
         self.g8_ws = None
         self.on_layer: Optional[Callable[[int, torch.Tensor], None]] = None
         self._zeros_h: Dict[int, torch.Tensor] = {}
+        self._split_for: set = set()    # (M, N, K) whose split product was timed faster
+        self._split_seen: set = set()
 
     # ------------------------------------------------------------------ weights
     def _read(self, path: str) -> dict:
@@ -156,6 +158,43 @@ class LatentDecoder:
         """Whether experts of these sizes run on the grouped matrix-core GEMMs."""
         return self.dtype == torch.bfloat16 and d * ff >= self.GROUPED_MIN and d % 64 == 0 and ff % 64 == 0 and ops.available()
 
+    # Few rows against a long reduction (a feed-forward's down projection in a decode step) leave most CUs idle in one GEMM:
+    # such a weight is kept a second time as S slices of the reduction [S, K / S, N] (S = 4, or 8 for at most 2048 outputs),
+    # run as ONE batched GEMM with fp32 partial products that the consumer adds up.  Which row counts take it is timed (tune_gemms).
+    SPLIT_ROWS, SPLIT_MIN_K = 256, 4096
+
+    def split_weight(self, w: torch.Tensor) -> Optional[torch.Tensor]:
+        """``w`` [N, K] in slices of the reduction, [S, K / S, N] (None where the split does not apply)."""
+        N, K = w.shape
+        S = 4 if N > 2048 else 8
+        if not self._mm32 or K < self.SPLIT_MIN_K or K % (8 * S) or N % 8:
+            return None
+        return w.t().contiguous().view(S, K // S, N)
+
+    @staticmethod
+    def _split_product(x: torch.Tensor, ws: torch.Tensor) -> torch.Tensor:
+        S, Ks, _ = ws.shape
+        return torch.bmm(x.view(x.shape[0], S, Ks).transpose(0, 1), ws, out_dtype=torch.float32)
+
+    def _linear_parts(self, x: torch.Tensor, w: torch.Tensor, ws: Optional[torch.Tensor]) -> torch.Tensor:
+        """x @ w^T as rows [M, N], or as fp32 partial products [S, M, N] where the split was timed faster for this M."""
+        if ws is not None and (x.shape[0], *w.shape) in self._split_for:
+            return self._split_product(x, ws)
+        return self._linear(x, w)
+
+    def _tune_split(self, M: int, w: torch.Tensor, ws: Optional[torch.Tensor]) -> None:
+        key = (M, *w.shape)
+        if ws is None or M > self.SPLIT_ROWS or key in self._split_seen:
+            return
+        self._split_seen.add(key)
+        x = torch.randn(M, w.shape[1], device=self.device).to(self.dtype)
+        t = {"one": [], "split": []}
+        for _ in range(5):
+            t["one"].append(gemm_plan._time(lambda: self._linear(x, w), iters=5, rounds=1))
+            t["split"].append(gemm_plan._time(lambda: self._split_product(x, ws), iters=5, rounds=1))
+        if sorted(t["split"])[2] < sorted(t["one"])[2]:
+            self._split_for.add(key)
+
     def tune_gemms(self, M: int, bucket: bool = False, lm_head: bool = True, only=None) -> None:
         """Pick the backend of the projections at M rows by timing the library and the hand-written cores (the engine
         calls this before it captures a decode bucket's graph).  bf16 only, and only where the full kernel extension is
@@ -169,6 +208,12 @@ class LatentDecoder:
             if w is not None and tuple(w.shape) not in seen and w.shape[0] % 8 == 0 and w.shape[1] % 8 == 0:
                 seen.add(tuple(w.shape))
                 gemm_plan.tune(torch.randn(M, w.shape[1], device=self.device).to(self.dtype), w, ws=self.g8_ws, bucket=bucket)
+        for w, ws in self._split_weights():
+            self._tune_split(M, w, ws)
+
+    def _split_weights(self) -> list:
+        """(weight, its split form or None) of the projections that :meth:`_linear_parts` runs."""
+        return []
 
     # ------------------------------------------------------------------ cache and state
     def latent_row_sizes(self, m) -> Tuple[int, int]:

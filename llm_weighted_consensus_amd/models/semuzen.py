@@ -45,6 +45,7 @@ class SemuzenLayer:
     w_o: torch.Tensor
     w_up: Optional[torch.Tensor] = None
     w_down: Optional[torch.Tensor] = None
+    w_down_split: Optional[torch.Tensor] = None
     extra: Dict[str, object] = field(default_factory=dict)
 
 
@@ -175,6 +176,7 @@ class SemuzenModel(LatentDecoder):
             subs.append(p + "{}1")
             if L.mlp is not None:
                 lay.w_up, lay.w_down = t(p + "mlp.up"), t(p + "mlp.down")
+                lay.w_down_split = self.split_weight(lay.w_down)
                 subs.append(p + "{}2")
             self.layers.append(lay)
         ones = torch.ones(cfg.streams, dtype=torch.float32, device=dev)
@@ -194,6 +196,9 @@ class SemuzenModel(LatentDecoder):
 
     def _gemm_weights(self) -> list:
         return [w for L in self.layers for w in (L.w_in, L.w_o, L.w_up, L.w_down)]
+
+    def _split_weights(self) -> list:
+        return [(L.w_down, L.w_down_split) for L in self.layers if L.w_down is not None]
 
     def _head(self) -> torch.Tensor:
         return self.head
@@ -277,7 +282,7 @@ class SemuzenModel(LatentDecoder):
             u, ff = self.updates[li]
             if ff is not None:
                 h = res32.hyper_step(X, y, u.coef, u.norm, dt, bias=u.bias)
-                y, u = self._linear(res32.relu2(self._linear(h, L.w_up)), L.w_down), ff
+                y, u = self._linear_parts(res32.relu2(self._linear(h, L.w_up)), L.w_down, L.w_down_split), ff
             if li + 1 < n:
                 h = res32.hyper_step(X, y, u.coef, u.norm, dt, bias=u.bias)
             if self.on_layer is not None:
@@ -288,7 +293,7 @@ class SemuzenModel(LatentDecoder):
     def _stream_sum(X: torch.Tensor, y: torch.Tensor, u: StreamUpdate) -> torch.Tensor:
         """The streams' sum behind an update that the forward pass leaves to the output rows (for ``on_layer``)."""
         X = X.clone()
-        res32.hyper_step(X, y, u.coef, u.norm, torch.float32 if y.dtype == torch.float32 else torch.bfloat16, bias=u.bias)
+        res32.hyper_step(X, y, u.coef, u.norm, y.dtype, bias=u.bias)
         return X.sum(0)
 
     def _output_rows(self, x, rows: Optional[torch.Tensor]) -> torch.Tensor:

@@ -106,7 +106,7 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
                 H: int, G: int, cu_q: Optional[torch.Tensor] = None, k_lens: Optional[torch.Tensor] = None,
                 max_q: int = 0, bias: Optional[torch.Tensor] = None, cores: Optional[bool] = None,
                 sink: Optional[torch.Tensor] = None, values_in_keys: bool = False, chunk: int = 0,
-                cap: float = 0.0) -> torch.Tensor:
+                cap: float = 0.0, splits: int = 0) -> torch.Tensor:
     """Sliding-window attention over the paged cache with the bias -r1_h ln(1 + r2_h (i - j)); ``q`` fp32
     [T, H*D] pre-scaled; row t reads table row t (``cu_q`` None) or the item whose ``cu_q`` range holds t.
     Over a bf16 cache whose sizes the matrix-core kernels are built for, prompt portions run on the portion kernel
@@ -119,7 +119,8 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
     values from the key rows.
     ``chunk`` > 0: positions are cut into chunks of that many, counted from position 0, and a row sees only keys of its
     own chunk (j >= i - i % chunk), besides the window.
-    ``cap`` > 0: a score becomes cap * tanh(score / cap), before the distance bias."""
+    ``cap`` > 0: a score becomes cap * tanh(score / cap), before the distance bias.
+    ``splits``: key ranges per decode row (0: chosen by the sizes)."""
     K = kernels()
     bs = k_cache.shape[1]
     D, Dv = k_cache.shape[2] // G, v_cache.shape[2] // G
@@ -127,7 +128,7 @@ def window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, p
     if cores and cu_q is None and positions.numel() > 0 and K.window_attn_decode_ok(D, Dv, bool(values_in_keys)):
         max_keys = min(int(window), block_tables.shape[1] * k_cache.shape[1], int(chunk) if chunk > 0 else 1 << 30)
         K.window_attn_decode(q, k_cache, v_cache, positions, block_tables, bias, int(window), max_keys, out, int(H), int(G),
-                             sink, bool(values_in_keys), int(chunk), float(cap))
+                             sink, bool(values_in_keys), int(chunk), float(cap), int(splits))
         return out
     if cores and cu_q is not None and k_lens is not None and max_q > 0 and K.window_attn_mfma_ok(D, Dv):
         K.window_attn_mfma(q, k_cache, v_cache, positions, cu_q, k_lens, int(max_q), block_tables, bias, int(window), out,
@@ -521,7 +522,7 @@ def embed_streams(table: torch.Tensor, tokens: torch.Tensor, scale: float, norm:
 
 def hyper_step(X: torch.Tensor, y: torch.Tensor, coef: torch.Tensor, nxt: Dyt, dtype, bias: Optional[torch.Tensor] = None,
                rows: Optional[torch.Tensor] = None, write: bool = True) -> torch.Tensor:
-    """A sublayer's result y (plus ``bias`` per column) into the streams X (fp32 [S, T, d], in place with ``write``):
+    """A sublayer's result y (rows [T, d], or planes [P, T, d] whose sum it is; plus ``bias`` per column) into the streams X (fp32 [S, T, d], in place with ``write``):
     X'_t = sum_s mix[s, t] X_s + out[t] y; returns h = nxt(sum_t in[t] X'_t) as ``dtype`` rows.  ``coef``:
     :func:`hyper_coef`.  ``rows`` (int64, needs write=False): only these rows of X and y."""
     n = X.shape[1] if rows is None else rows.numel()

@@ -73,6 +73,39 @@ def test_streams_update_and_next_norm(gpu, S, d, act, ydt):
             assert torch.equal(Xg.cpu(), X) and ((h.cpu().double() - hr[rows or slice(None)]).abs() < lim[rows or slice(None)]).all()
 
 
+@pytest.mark.parametrize("S,d,P", [(2, 64, 4), (3, 46, 2), (6, 40, 3)])
+def test_streams_update_from_partial_products(gpu, S, d, P):
+    """The result as planes of a split GEMM: their sum enters the streams."""
+    from llm_weighted_consensus_amd.ops import res32
+
+    g = torch.Generator().manual_seed(d)
+    X, y = torch.randn(S, 5, d, generator=g), torch.randn(P, 5, d, generator=g)
+    coef, bias = torch.randn(S * S + 2 * S, generator=g).to(gpu), torch.randn(d, generator=g).to(gpu)
+    nxt, _ = _dyt(d, g, gpu, 0.7)
+    a, b = X.to(gpu), X.to(gpu)
+    ha = res32.hyper_step(a, y.to(gpu), coef, nxt, BF16, bias=bias)
+    hb = res32.hyper_step(b, y.to(gpu).sum(0), coef, nxt, BF16, bias=bias)
+    assert (a - b).abs().max() < 1e-5 * S and (ha.float() - hb.float()).abs().max() < 0.05
+    rows = torch.tensor([4, 1], device=gpu)
+    assert torch.equal(res32.hyper_step(X.to(gpu), y.to(gpu), coef, nxt, BF16, bias=bias, rows=rows, write=False), ha[rows])
+
+
+def test_split_down_projection(gpu, tmp_path):
+    """A feed-forward wide enough for the split form: decode steps with it (forced) and without give the oracle's logits."""
+    cfg = O.make_config(64, 90, [O.attention_layer(2, 1, 16, 16, 4096), O.latent_layer(2, 16, 8, 16, 32, 9, 4160)], streams=2)
+    W = O.make_weights(cfg, 2)
+    model, eng = _engine(_save(tmp_path / "m", cfg, W), 90, BF16)
+    pairs = model._split_weights()
+    assert len(pairs) == 2 and all(s is not None and s.shape == (8, w.shape[1] // 8, 64) for w, s in pairs)
+    toks = _tokens(30, 90, 3)
+    ref = O.forward(cfg, W, toks)
+    for forced in (False, True):
+        model._split_for = {(1, *w.shape) for w, _ in pairs} if forced else set()
+        got = [eng.step_tokens([("s", toks[:20], list(range(20)))])]
+        got += [eng.step_tokens([("s", [t], [0])], ["s"] if i == 9 else []) for i, t in enumerate(toks[20:])]
+        assert _err(torch.cat(got), ref, BF16) < TOL[BF16]
+
+
 @pytest.mark.parametrize("dtype,tol", DTYPES)
 @pytest.mark.parametrize("S,d", [(1, 46), (3, 64), (6, 40)])
 def test_streams_start_as_the_normed_embedding(gpu, S, d, dtype, tol):
